@@ -18,7 +18,7 @@ from typing import Optional
 @dataclass
 class ModelConfig:
     name: str
-    arch: str  # "llama" | "qwen3" | "mixtral" | "voletar" | "tapasun" | "momuvik" | "seradra"
+    arch: str  # "llama" | "qwen3" | "mixtral" | "voletar" | "tapasun" | "momuvik" | "seradra" | "tarorax"
     hidden_size: int
     intermediate_size: int
     num_layers: int
@@ -40,7 +40,7 @@ class ModelConfig:
     bos_token_id: Optional[int] = None
     eos_token_ids: list = field(default_factory=list)
     chat_template: str = "llama3"
-    # designs whose config lists their layers (arch "voletar", "tapasun", "momuvik", "seradra"): the checkpoint's own
+    # designs whose config lists their layers (arch "voletar", "tapasun", "momuvik", "seradra", "tarorax"): the checkpoint's own
     # config.json structure -- per-layer mixer type and sizes, norm eps and the design's other
     # constants -- as the design's module (mxserve/models/<arch>.py) reads it.  None for the uniform
     # transformer families.
@@ -52,10 +52,10 @@ class ModelConfig:
 
     @property
     def has_recurrent_state(self) -> bool:
-        """Layers that carry a per-sequence state from token to token (linear attention, mLSTM, state
-        spaces, delta rule, short convolutions): no prefix caching (a cached block has no state to
+        """Layers that carry a per-sequence state from token to token (linear attention, gated or not, mLSTM,
+        state spaces, delta rule, short convolutions): no prefix caching (a cached block has no state to
         resume from) and one state slot per request."""
-        return self.arch in ("voletar", "tapasun")
+        return self.arch in ("voletar", "tapasun", "tarorax")
 
     @property
     def q_size(self) -> int:
@@ -333,7 +333,43 @@ _reg(seradra_config("tiny-seradra", {
          "mixer": dict(_latent(4, 16, 8, 24, 32, 40, 0.2), mask={"size": 33})}]}))
 
 
+def tarorax_config(name: str, d: dict) -> ModelConfig:
+    """A Tarorax checkpoint's config.json: `width`, `vocab`, `streams`, `norm.eps`, `layers` (each with `type` gla |
+    attention, `mixer`, `mlp` dense | moe | null).  The uniform fields are filled from the first layer for the
+    code that sizes things from them."""
+    layers = d["layers"]
+    att = layers[0]["mixer"] if layers else {"heads": 1, "dim": int(d["width"])}
+    ffs = [int(l["mlp"]["ff"]) if l["mlp"].get("kind", "dense") == "dense" else int(l["mlp"]["expert"]["ff"])
+           for l in layers if l.get("mlp")]
+    moes = [l["mlp"]["router"] for l in layers if l.get("mlp") and l["mlp"].get("kind") == "moe"]
+    keep = {k: d[k] for k in ("layers", "norm", "streams", "width", "vocab") if k in d}
+    return ModelConfig(
+        name=name, arch="tarorax", hidden_size=int(d["width"]), intermediate_size=max(ffs) if ffs else 0,
+        num_layers=len(layers), num_heads=int(att["heads"]), num_kv_heads=int(att.get("kv_heads", att["heads"])),
+        head_dim=int(att["dim"]), vocab_size=int(d["vocab"]),
+        rms_norm_eps=float((d.get("norm") or {}).get("eps", 1e-5)), tie_word_embeddings=True,
+        max_position_embeddings=int(d.get("max_position_embeddings", 1 << 20)),
+        num_experts=max((int(r["experts"]) for r in moes), default=0),
+        num_experts_per_tok=max((int(r["top"]) for r in moes), default=0),
+        bos_token_id=d.get("bos_token_id"), eos_token_ids=list(d.get("eos_token_ids") or []),
+        chat_template="chatml", arch_config=keep)
+
+
+# A small Tarorax (random weights): both mixers, a dense and a routed feed-forward, a layer without one.
+_reg(tarorax_config("tiny-tarorax", {
+    "architecture": "Tarorax", "width": 96, "vocab": 384, "norm": {"eps": 1e-5}, "streams": 3,
+    "layers": [
+        {"type": "gla", "mlp": {"kind": "dense", "ff": 160}, "mixer": {"heads": 3, "dim": 16, "vdim": 24, "tau": 8.0}},
+        {"type": "attention", "mixer": {"heads": 4, "kv_heads": 2, "dim": 16, "vdim": 32, "scale": 0.25, "softcap": 20.0,
+                                        "diff": 0.4, "conv": 3, "q_temp": {"coef": 0.2, "every": 32}},
+         "mlp": {"kind": "moe", "expert": {"ff": 48},
+                 "router": {"experts": 12, "top": 3, "groups": {"count": 4, "keep": 2}, "scale": 1.5}}},
+        {"type": "gla", "mlp": None, "mixer": {"heads": 2, "dim": 40, "vdim": 32, "tau": 16.0}}]}))
+
+
 def _from_hf_json(name: str, d: dict) -> ModelConfig:
+    if d.get("architecture") == "Tarorax":
+        return tarorax_config(name, d)
     if d.get("architecture") == "Seradra":
         return seradra_config(name, d)
     if d.get("architecture") == "Momuvik":

@@ -2,16 +2,18 @@
 constants as parameters.  Like the mixers (mxserve/models/mixers.py) they name their checkpoint
 tensors, re-pack them once when the weights are loaded, and compute from a step's flattened batch.
 
-  GatedFF        W_down(act(W_gate h) * W_up h), gate and up as one projection; act = silu
+  GatedFF        W_down(act(W_gate h) * W_up h), gate and up as one projection; act = silu, or a gelu in its
+                 exact or its tanh form
   CurvedFF       W_down(act(W_up h)) without a gate; act is a parabola above zero and an exponential
                  below it, with two learned numbers (`<p>act`)
   CappedExpert   one small gated unit with clipped pre-activations: g = min(W_gate x, limit),
                  u = clamp(W_up x, -limit, limit), W_down(g * sigmoid(alpha g) * (u + 1))
   RoutedExperts  a router (fp32; sigmoid scores, or a softmax over all experts) picks `top` of `experts`
-                 small gated units per token (CappedExperts, or plain SiLU units when no limit is
-                 given); the chosen scores (optionally renormalised) weigh each expert's INPUT or its
-                 OUTPUT; an optional shared CappedExpert with its own size and limit sees every token
-                 unweighted
+                 small units per token (CappedExperts, or plain gated units when no limit is given, or
+                 ungated W_down(act(W_up h))); the choice may add a learned correction to the scores and
+                 be limited to the best groups of experts; the chosen scores (optionally renormalised and
+                 scaled) weigh each expert's INPUT or its OUTPUT; an optional shared CappedExpert with its
+                 own size and limit sees every token unweighted
 
 The kernels are in mxserve/ops/seqmix.py (csrc/mixers/latent_experts.hip on the GPU); the matrix products go
 through ops.linear and torch.bmm (hipBLASLt).
@@ -39,8 +41,10 @@ class FeedForward:
 
 
 class GatedFF(FeedForward):
-    def __init__(self, prefix: str, width: int, ff: int):
-        self.p, self.width, self.ff = prefix, width, int(ff)
+    def __init__(self, prefix: str, width: int, ff: int, act: str = "silu"):
+        if act not in seqmix.ACTS:
+            raise ValueError(f"{prefix}: unknown activation {act!r}")
+        self.p, self.width, self.ff, self.act = prefix, width, int(ff), act
 
     def shapes(self) -> dict:
         p = self.p
@@ -52,7 +56,9 @@ class GatedFF(FeedForward):
 
     def forward(self, h: torch.Tensor, w: dict) -> torch.Tensor:
         p = self.p
-        return ops.linear(seqmix.silu_mul(ops.linear(h, w[p + "_gu"])), w[p + "down"])
+        gu = ops.linear(h, w[p + "_gu"])
+        a = seqmix.silu_mul(gu) if self.act == "silu" else seqmix.act_mul(gu, self.act)
+        return ops.linear(a, w[p + "down"])
 
 
 class CurvedFF(FeedForward):
@@ -94,11 +100,12 @@ class CappedExpert(FeedForward):
 
 
 class RoutedExperts(FeedForward):
-    """Tensors: `<p>router` [E, width], `<p>e<i>.{gate,up,down}`, optionally `<p>shared.{gate,up,down}`.
-    Loaded as `<p>_gu` [E, 2 ff, width] and `<p>_down` [E, width, ff].
+    """Tensors: `<p>router` [E, width], `<p>e<i>.{gate,up,down}` (ungated: no gate), optionally `<p>correction` [E]
+    and `<p>shared.{gate,up,down}`.  Loaded as `<p>_in` [E, width, 2 ff] (ungated: [E, width, ff]) and `<p>_down`
+    [E, ff, width], the right-hand operands of the batched products as they are (never a transposed view).
 
     Two ways through the experts, both exact (a token never meets an expert it did not choose with
-    anything but a zero row, and a zero row gives a zero output: g = 0):
+    anything but a zero row, and a zero row gives a zero output):
       batched   every expert over all T rows of `spread_scaled` in two batched products -- no sorting
                 and no host round trip, so a captured single-token step can replay it; E / top times
                 the needed products, which steps of a few tokens do not feel (they stream the
@@ -112,27 +119,43 @@ class RoutedExperts(FeedForward):
 
     def __init__(self, prefix: str, width: int, experts: int, top: int, ff: int, limit: Optional[float],
                  shared: Optional[CappedExpert] = None, alpha: float = 1.702, renorm: bool = False,
-                 score: str = "sigmoid", weigh: str = "input"):
-        """limit None: an expert is W_down(SiLU(W_gate x) * W_up x).  score: sigmoid | softmax (over all
-        experts, before the choice).  weigh: input | output (what a chosen score multiplies)."""
+                 score: str = "sigmoid", weigh: str = "input", gated: bool = True, act: str = "silu",
+                 correction: bool = False, groups: int = 1, keep: int = 1, scale: float = 1.0):
+        """limit None: an expert is W_down(act(W_gate x) * W_up x), or W_down act(W_up x) when not `gated`.  score:
+        sigmoid | softmax (over all experts, before the choice).  weigh: input | output (what a chosen score
+        multiplies).  correction: a tensor added to the scores for the choice only.  groups, keep: the choice is
+        limited to the `keep` best of so many groups of neighbours.  renorm, scale: the weights are the chosen
+        scores, divided by their sum, times scale."""
         if not 1 <= top <= experts:
             raise ValueError(f"{prefix}: top {top} of {experts} experts")
-        if score not in ("sigmoid", "softmax") or weigh not in ("input", "output"):
-            raise ValueError(f"{prefix}: score {score!r}, weigh {weigh!r}")
+        if score not in ("sigmoid", "softmax") or weigh not in ("input", "output") or act not in seqmix.ACTS:
+            raise ValueError(f"{prefix}: score {score!r}, weigh {weigh!r}, act {act!r}")
+        if groups < 1 or experts % groups or not 1 <= keep <= groups or top > keep * (experts // groups):
+            raise ValueError(f"{prefix}: top {top} of {experts} experts in {keep} of {groups} groups")
+        if limit is not None and not gated:
+            raise ValueError(f"{prefix}: capped experts are gated")
         self.p, self.width, self.E, self.top, self.ff = prefix, width, int(experts), int(top), int(ff)
         self.limit = None if limit is None else float(limit)
         self.alpha, self.renorm, self.shared = float(alpha), bool(renorm), shared
         self.softmax, self.on_output = score == "softmax", weigh == "output"
+        self.gated, self.act_kind, self.correction = bool(gated), act, bool(correction)
+        self.groups, self.keep, self.scale = int(groups), int(keep), float(scale)
 
     def act(self, gu: torch.Tensor) -> torch.Tensor:
+        if not self.gated:
+            return seqmix.unary_act(gu, self.act_kind)
         if self.limit is None:
-            return seqmix.silu_mul(gu)
+            return seqmix.silu_mul(gu) if self.act_kind == "silu" else seqmix.act_mul(gu, self.act_kind)
         return seqmix.capped_glu(gu, self.limit, self.alpha)
 
     def shapes(self) -> dict:
         p, sh = self.p, {self.p + "router": (self.E, self.width)}
+        if self.correction:
+            sh[p + "correction"] = (self.E,)
         for e in range(self.E):
-            sh[f"{p}e{e}.gate"] = sh[f"{p}e{e}.up"] = (self.ff, self.width)
+            if self.gated:
+                sh[f"{p}e{e}.gate"] = (self.ff, self.width)
+            sh[f"{p}e{e}.up"] = (self.ff, self.width)
             sh[f"{p}e{e}.down"] = (self.width, self.ff)
         if self.shared is not None:
             sh.update(self.shared.shapes())
@@ -140,26 +163,31 @@ class RoutedExperts(FeedForward):
 
     def finish_weights(self, w: dict) -> None:
         p = self.p
-        w[p + "_gu"] = torch.stack([torch.cat([w.pop(f"{p}e{e}.gate"), w.pop(f"{p}e{e}.up")]) for e in range(self.E)]).contiguous()
-        w[p + "_down"] = torch.stack([w.pop(f"{p}e{e}.down") for e in range(self.E)]).contiguous()
+        names = ("gate", "up") if self.gated else ("up",)
+        w[p + "_in"] = torch.stack([torch.cat([w.pop(f"{p}e{e}.{n}") for n in names]).t() for e in range(self.E)]).contiguous()
+        w[p + "_down"] = torch.stack([w.pop(f"{p}e{e}.down").t() for e in range(self.E)]).contiguous()
+        if self.correction:
+            w[p + "correction"] = w[p + "correction"].to(torch.float32).contiguous()
         if self.shared is not None:
             self.shared.finish_weights(w)
 
     def route(self, h: torch.Tensor, w: dict) -> tuple:
         logits = seqmix.gate_linear(h, w[self.p + "router"], None)  # fp32 products and sums
-        return seqmix.route_topk(logits, self.top, self.renorm, self.softmax)
+        return seqmix.route_topk(logits, self.top, self.renorm, self.softmax,
+                                 correction=w[self.p + "correction"] if self.correction else None, groups=self.groups,
+                                 keep=self.keep, scale=self.scale)
 
     def forward(self, h: torch.Tensor, w: dict) -> torch.Tensor:
         p, T = self.p, h.shape[0]
         tw, ids = self.route(h, w)
         w_in, w_out = (None, tw) if self.on_output else (tw, None)
         extra = self.shared.forward(h, w) if self.shared is not None else None
-        gu, down = w[p + "_gu"], w[p + "_down"]
+        up, down = w[p + "_in"], w[p + "_down"]
         capturing = h.is_cuda and torch.cuda.is_current_stream_capturing()
         if T <= self.BATCHED_MAX_TOKENS or T * self.E <= self.BATCHED_MAX_ROWS or capturing:
             xs = seqmix.spread_scaled(h, w_in, ids, self.E)  # [E, T, W]
-            a = self.act(torch.bmm(xs, gu.transpose(1, 2)).view(self.E * T, -1))
-            ys = torch.bmm(a.view(self.E, T, -1), down.transpose(1, 2))  # [E, T, W]
+            a = self.act(torch.bmm(xs, up).view(self.E * T, -1))
+            ys = torch.bmm(a.view(self.E, T, -1), down)  # [E, T, W]
             if w_out is None:
                 return seqmix.expert_combine(ys, None, self.E, T, extra, row_stride=T)
             # weights on the outputs: a token's k chosen slabs, row (expert, t) of the stack
@@ -171,5 +199,5 @@ class RoutedExperts(FeedForward):
         for e in range(self.E):
             a0, a1 = o[e], o[e + 1]
             if a1 > a0:
-                ys[a0:a1] = ops.linear(self.act(ops.linear(xs[a0:a1], gu[e])), down[e])
+                torch.mm(self.act(torch.mm(xs[a0:a1], up[e])), down[e], out=ys[a0:a1])
         return seqmix.expert_combine(ys, inv, self.top, T, extra, weights=w_out)

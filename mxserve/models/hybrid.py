@@ -1,6 +1,6 @@
 """What the designs whose config lists their layers share (mxserve/models/voletar.py,
-mxserve/models/tapasun.py, mxserve/models/momuvik.py, mxserve/models/seradra.py): the plan of layer runs with every run's place inside a cache block and a
-state slot, and the model surface the runner expects (weights in a flat dict, the mixers' input
+mxserve/models/tapasun.py, mxserve/models/momuvik.py, mxserve/models/seradra.py, mxserve/models/tarorax.py):
+the plan of layer runs with every run's place inside a cache block and a state slot, and the model surface the runner expects (weights in a flat dict, the mixers' input
 projections fused into one GEMM per layer, cache geometry from the plan).
 
 A design's module provides `mixers_of(ac)` (its config's layers as mxserve/models/mixers.py objects),
@@ -18,7 +18,7 @@ from ..parallel.comm import get_tp
 from .config import ModelConfig
 from .mixers import Mixer
 
-HYBRID_ARCHS = ("voletar", "tapasun", "momuvik", "seradra")
+HYBRID_ARCHS = ("voletar", "tapasun", "momuvik", "seradra", "tarorax")
 
 
 def design_module(arch: str):

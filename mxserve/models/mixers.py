@@ -31,6 +31,12 @@ in a slot) and computes its output from a step's flattened token batch.
                         the softmax; projections with biases, one RMS norm over all query rows and one
                         over all key rows, half-split rotary pairs on part of each head with
                         ramp-blended frequencies and a factor on cos / sin, sliding window, learned sink
+  DifferentialAttention softmax attention in two maps over the same values, the second subtracted a learned
+                        number of times from the first; biased projections, short convolutions on q, k and v,
+                        a query factor that grows with the position, bounded scores, unit norm per head, and
+                        a sigmoid output gate; no rotation
+  GatedLinearAttention  S = diag(a) S + k v^T, o = S^T q with a decay per head and key channel from a low-rank
+                        pair, per-head RMS norm and a SiLU output gate
 
 The kernels are in mxserve/ops/seqmix.py (csrc/mixers/*.hip on the GPU).
 """
@@ -59,6 +65,7 @@ class StepContext:
 class Mixer:
     kv_heads = dk = dv = 0  # paged K/V per token (0: none)
     state_floats = 0  # fp32 state per sequence
+    out_bias: Optional[str] = None  # tensor that the layer adds to forward()'s result
 
     def proj_rows(self) -> list:
         """[(tensor name, rows)] of the fused input projection, in the order forward() reads them."""
@@ -621,6 +628,105 @@ class TalkingAttention(Mixer):
                                     0, md.max_query_len, sink=w.get(p + "sink"), talk=w.get(p + "talk"),
                                     max_seq_len=getattr(md, "max_seq_len", 0))
         return ops.linear(o, w[p + "o"])
+
+
+class DifferentialAttention(Mixer):
+    """Per head two queries and two keys of size dim (q has H * 2 * dim rows, k has G * 2 * dim, head by head as
+    [map 1 | map 2]) over one value of size vdim.
+        q, k, v: projections with biases, then a causal filter of `conv` taps on every channel
+        q <- q * (1 + temp.coef * ln(floor((p + 1) / temp.every) + 1)) at position p
+        a_m = softmax(softcap * tanh(scale q_m . k_m / softcap)) V,   o = a_1 - lambda a_2
+        lambda = exp(lq1 . lk1) - exp(lq2 . lk2) + diff, one number for the layer
+        o / rms(o) * (1 - diff) per head, times sigmoid(W_g h), output projection with a bias
+    The pages hold a kv head's two keys side by side.  State per sequence: the filter's last conv - 1 inputs
+    (projected values with their biases; q, k and v in one block)."""
+
+    def __init__(self, prefix: str, width: int, heads: int, kv_heads: int, dim: int, vdim: int, scale: float,
+                 diff: float, softcap: float, conv: int, temp: Optional[dict] = None):
+        if heads % kv_heads or conv < 1:
+            raise ValueError(f"{prefix}: {heads} query heads over {kv_heads} kv heads, {conv} taps")
+        self.p, self.width = prefix, width
+        self.heads, self.kv_heads, self.qk, self.dv = heads, kv_heads, dim, vdim
+        self.dk = 2 * dim  # a page row: both maps' keys
+        self.scale, self.diff, self.softcap, self.taps = float(scale), float(diff), float(softcap), int(conv)
+        self.temp_coef = float(temp["coef"]) if temp else 0.0
+        self.temp_every = float(temp["every"]) if temp else 1.0
+        self.q_cols = heads * 2 * dim
+        self.conv_ch = self.q_cols + kv_heads * (2 * dim + vdim)
+        self.state_floats = -(-(conv - 1) * self.conv_ch // 4) * 4
+        self.out_bias = prefix + "o.b"
+        self.lam = diff  # from the tensors when they are loaded
+
+    def proj_rows(self) -> list:
+        p, G = self.p, self.kv_heads
+        return [(p + "q", self.q_cols), (p + "k", G * self.dk), (p + "v", G * self.dv), (p + "g", self.heads * self.dv)]
+
+    def extra_shapes(self) -> dict:
+        p, sh = self.p, {}
+        for n, rows in (("q", self.q_cols), ("k", self.kv_heads * self.dk), ("v", self.kv_heads * self.dv)):
+            sh[p + n + ".b"] = (rows,)
+            sh[p + n + ".conv"] = (rows, self.taps)
+        for n in ("lq1", "lk1", "lq2", "lk2"):
+            sh[p + n] = (self.qk,)
+        sh[p + "o"] = (self.width, self.heads * self.dv)
+        sh[p + "o.b"] = (self.width,)
+        return sh
+
+    def finish_weights(self, w: dict) -> None:
+        p = self.p
+        # one filter and one bias over q, k, v's channels; the filter tap-major for the kernel
+        w[p + "_conv"] = torch.cat([w.pop(p + n + ".conv") for n in "qkv"]).t().contiguous()
+        w[p + "_b"] = torch.cat([w.pop(p + n + ".b") for n in "qkv"]).contiguous()
+        d = [float((w.pop(p + "lq" + n).double() * w.pop(p + "lk" + n).double()).sum()) for n in "12"]
+        self.lam = math.exp(d[0]) - math.exp(d[1]) + self.diff
+
+    def forward(self, parts: list, h: torch.Tensor, w: dict, ctx: StepContext, koff: int, voff: int, soff: int):
+        md, p, G = ctx.md, self.p, self.kv_heads
+        q, g = parts[0], parts[3]
+        # q, k, v are neighbours in the fused projection (proj_rows)
+        qkv = torch.as_strided(q, (q.shape[0], self.conv_ch), q.stride(), q.storage_offset())
+        qc = seqmix.conv_qkv_cache(qkv, w[p + "_conv"], w[p + "_b"], ctx.state, md.state_rows, soff, md.query_start_loc,
+                                   md.seq_lens, md.positions, md.slot_mapping, ctx.cache, koff, voff, self.q_cols, G,
+                                   self.dk, self.dv, ctx.block_size, self.temp_coef, self.temp_every, md.max_query_len)
+        o = seqmix.differential_attention(qc, ctx.cache, md.block_tables, md.query_start_loc, md.seq_lens, koff, voff,
+                                          self.heads, G, self.qk, self.dv, ctx.block_size, self.scale, self.softcap,
+                                          self.lam, 1.0 - self.diff, ctx.eps, g, md.max_query_len,
+                                          getattr(md, "max_seq_len", 0), getattr(md, "num_decodes", 0))
+        return ops.linear(o, w[p + "o"])
+
+
+class GatedLinearAttention(Mixer):
+    """q = W_q h * dim^-1/2 and k = W_k h per head, v = W_v h; decay sigmoid(W_a2 (W_a1 h) + b)^(1/tau) per head and
+    key channel; S <- diag(decay) S + k v^T, o = S^T q; RMS norm of every head's o with a weight shared by the
+    heads, times SiLU(W_g h), output projection.  State per sequence: S, stored [heads, vdim, dim]."""
+
+    def __init__(self, prefix: str, width: int, heads: int, dim: int, vdim: int, tau: float):
+        self.p, self.width = prefix, width
+        self.heads, self.qk, self.vd, self.tau = heads, dim, vdim, float(tau)
+        self.state_floats = -(-heads * dim * vdim // 4) * 4
+        self.rank = 16  # no config entry: a checkpoint's tensors give it; this is what random weights are made with
+
+    def adopt_shapes(self, full: dict) -> None:
+        a1 = full.get(self.p + "a1")
+        if a1 is not None and a1.dim() == 2:
+            self.rank = int(a1.shape[0])
+
+    def proj_rows(self) -> list:
+        p, n, m = self.p, self.heads * self.qk, self.heads * self.vd
+        return [(p + "q", n), (p + "k", n), (p + "v", m), (p + "g", m), (p + "a1", self.rank)]
+
+    def extra_shapes(self) -> dict:
+        p, n = self.p, self.heads * self.qk
+        return {p + "a2": (n, self.rank), p + "a2.b": (n,), p + "norm": (self.vd,), p + "o": (self.width, self.heads * self.vd)}
+
+    def forward(self, parts: list, h: torch.Tensor, w: dict, ctx: StepContext, koff: int, voff: int, soff: int):
+        q, k, v, g, a1 = parts
+        md, p, H = ctx.md, self.p, self.heads
+        loga = seqmix.decay_lowrank(a1, w[p + "a2"], w[p + "a2.b"], self.tau)
+        o = seqmix.gla_scan(q, k, v, loga, ctx.state, md.state_rows, soff, md.query_start_loc, md.seq_lens, H, self.qk,
+                            self.vd, self.qk ** -0.5, max_query_len=md.max_query_len)
+        y = seqmix.gated_norm(o, g, w[p + "norm"], ctx.eps, H, "silu", False, h.dtype)
+        return ops.linear(y, w[p + "o"])
 
 
 def build_mixer(kind: str, prefix: str, width: int, mc: dict) -> Mixer:

@@ -1,6 +1,7 @@
 """Sequence-mixer ops beyond rotary softmax attention: a 32-bit residual stream with fused norms,
-paged attention with a sliding window and kept first tokens, decayed linear attention, the mLSTM
-matrix memory, gated output norms, squared ReLU and logit soft-capping.
+paged attention with a sliding window and kept first tokens, attention in two subtracted maps, decayed and
+gated linear attention, the mLSTM matrix memory, several residual streams, gated output norms, squared ReLU
+and logit soft-capping.
 
 Like mxserve.ops: GPU tensors run the gfx950 kernels of the in-tree extension `mxserve/_M*.so`
 (csrc/mixers/*.hip, activations bf16 or fp32; built by `python setup_ext.py --only M` or on first
@@ -15,7 +16,7 @@ Paged cache of one attention layer inside the block-major pool `cache` [num_bloc
 K at `koff` as [Hkv, BS, dk], V at `voff` as [Hkv, BS, dv], both token-major.
 Recurrent state of one layer inside the slot pool `state` [slots, state_floats] (fp32): decayed
 linear attention S [H, dk, dv] at `off`; mLSTM S [H, dk, dv], then n [H, dk], then m [H]; the
-column scans (state-space duality, gated delta rule) S transposed [H, dv, dk], so that the rows a
+column scans (state-space duality, gated delta rule, gated linear attention) S transposed [H, dv, dk], so that the rows a
 lane owns are contiguous; a short causal convolution its last taps - 1 inputs [taps - 1, channels].
 """
 from __future__ import annotations
@@ -142,6 +143,49 @@ def cast_into(dst: torch.Tensor, x: torch.Tensor) -> None:
         dst[:, :x.shape[1]].copy_(x)
 
 
+# ----------------------------------------------------------------------------- several residual streams
+def streams_start(ids: torch.Tensor, table: torch.Tensor, streams: int, w_in: torch.Tensor, norm_w: torch.Tensor,
+                  eps: float, w_offset: float, out_dtype: torch.dtype) -> tuple:
+    """n = `streams` residual streams that all begin as the embedding.  w_in fp32 [n]: what the first sublayer
+    reads is u = sum_s w_in[s] x_s.  -> (X fp32 [T, n, W], RMSNorm(u) * (w_offset + norm_w) in out_dtype)."""
+    T, W = ids.shape[0], table.shape[1]
+    if _gpu(table):
+        X = torch.empty(T, streams, W, dtype=torch.float32, device=table.device)
+        h = torch.empty(T, W, dtype=out_dtype, device=table.device)
+        ext().streams_start(X, h, ids, table, w_in, norm_w, float(eps), float(w_offset))
+        return X, h
+    e = F.embedding(ids, table).float()
+    X = e.unsqueeze(1).expand(T, streams, W).contiguous()
+    u = torch.einsum("s,tsw->tw", w_in, X)
+    return X, (_rms(u, eps) * (norm_w.float() + w_offset)).to(out_dtype)
+
+
+def streams_update(X: torch.Tensor, y: torch.Tensor, coeffs: torch.Tensor, eps: float, norm_w: torch.Tensor,
+                   out_dtype: torch.dtype, *, bias: Optional[torch.Tensor] = None,
+                   scale: Optional[torch.Tensor] = None, w_offset: float = 0.0) -> torch.Tensor:
+    """One pass over n fp32 residual streams X [T, n, W], in place, all streams at once from the old ones:
+        d = (y + bias) * scale          (bias, scale [W]; either may be absent)
+        x_t <- sum_s mix[s, t] x_s + w_out[t] d
+    and the next sublayer's input, RMSNorm(sum_s w_in[s] x_s) * (w_offset + norm_w) of the new streams, in
+    out_dtype.  coeffs fp32 [n * n + 2 n] = mix ([from, to], row-major) | w_out | w_in.  All sums in fp32."""
+    n = X.shape[1]
+    if coeffs.numel() != n * n + 2 * n:
+        raise ValueError(f"streams_update: {coeffs.numel()} coefficients for {n} streams")
+    if _gpu(X):
+        h = torch.empty(X.shape[0], X.shape[2], dtype=out_dtype, device=X.device)
+        ext().streams_update(X, y, bias, scale, coeffs, norm_w, h, float(eps), float(w_offset))
+        return h
+    d = y.float()
+    if bias is not None:
+        d = d + bias.float()
+    if scale is not None:
+        d = d * scale.float()
+    mix, w_out, w_in = coeffs[:n * n].view(n, n), coeffs[n * n:n * n + n], coeffs[n * n + n:]
+    X.copy_(torch.einsum("st,bsw->btw", mix, X) + w_out.view(1, n, 1) * d.unsqueeze(1))
+    u = torch.einsum("s,tsw->tw", w_in, X)
+    return (_rms(u, eps) * (norm_w.float() + w_offset)).to(out_dtype)
+
+
 def relu_sq(x: torch.Tensor) -> torch.Tensor:
     """max(x, 0)^2, computed in fp32."""
     if _gpu(x):
@@ -161,6 +205,34 @@ def xielu(x: torch.Tensor, ab: torch.Tensor) -> torch.Tensor:
     z = x.float()
     zn = z.clamp(max=0.0)
     return torch.where(z > 0, ab[0] * z * z + 0.5 * z, ab[1] * (torch.expm1(zn) - zn) + 0.5 * z).to(x.dtype)
+
+
+ACTS = {"silu": 0, "gelu_erf": 1, "gelu_tanh": 2}
+
+
+def _act(z: torch.Tensor, kind: str) -> torch.Tensor:
+    if kind == "silu":
+        return F.silu(z)
+    return F.gelu(z, approximate="tanh" if kind == "gelu_tanh" else "none")
+
+
+def unary_act(x: torch.Tensor, kind: str) -> torch.Tensor:
+    """act(x) with kind in silu | gelu_erf (the exact form) | gelu_tanh; computed in fp32."""
+    if _gpu(x):
+        out = torch.empty_like(x)
+        ext().unary_act(out, x, ACTS[kind])
+        return out
+    return _act(x.float(), kind).to(x.dtype)
+
+
+def act_mul(gu: torch.Tensor, kind: str) -> torch.Tensor:
+    """act(gu[:, :F]) * gu[:, F:] of a fused gate/up projection [T, 2F]; fp32 inside."""
+    Fh = gu.shape[1] // 2
+    if _gpu(gu):
+        out = torch.empty(gu.shape[0], Fh, dtype=gu.dtype, device=gu.device)
+        ext().act_mul(out, gu, ACTS[kind])
+        return out
+    return (_act(gu[:, :Fh].float(), kind) * gu[:, Fh:].float()).to(gu.dtype)
 
 
 def softcap(x: torch.Tensor, cap: float) -> torch.Tensor:
@@ -541,7 +613,148 @@ def causal_conv(x: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor], 
     return (F.silu(out) if silu else out).to(x.dtype)
 
 
+def conv_qkv_cache(x: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor], state: torch.Tensor,
+                   state_rows: torch.Tensor, off: int, qsl: torch.Tensor, seq_lens: torch.Tensor,
+                   positions: torch.Tensor, slot_mapping: torch.Tensor, cache: torch.Tensor, koff: int, voff: int,
+                   q_cols: int, num_kv_heads: int, dk: int, dv: int, block_size: int, temp_coef: float = 0.0,
+                   temp_every: float = 1.0, max_query_len: int = 0) -> torch.Tensor:
+    """Queries, keys and values of a step from the fused projection to what attention reads, for a mixer whose
+    q, k, v pass a short causal filter: u = x + bias (x [T, q_cols + G*dk + G*dv], a row-strided view),
+    y[t, c] = sum_j w[j, c] u[t - (taps-1) + j, c] as in causal_conv (no bias after it, no activation; the carried
+    inputs are u).  Query columns are multiplied by 1 + temp_coef * ln(floor((p + 1) / temp_every) + 1) at position
+    p and returned [T, q_cols]; keys and values go into the paged cache (slot -1: not written).  fp32 inside, one
+    rounding at the end."""
+    T, C = x.shape
+    if C != q_cols + num_kv_heads * (dk + dv):
+        raise ValueError(f"conv_qkv_cache: {C} columns for {q_cols} query, {num_kv_heads} x ({dk} + {dv}) key / value")
+    if _gpu(x):
+        q = torch.empty(T, q_cols, dtype=x.dtype, device=x.device)
+        ext().conv_qkv_cache(q, x, w, bias, state, state_rows, int(off), qsl, seq_lens, positions, slot_mapping, cache,
+                             int(koff), int(voff), num_kv_heads, dk, dv, block_size, float(temp_coef), float(temp_every),
+                             int(max_query_len))
+        return q
+    u = x.float() if bias is None else x.float() + bias.float()
+    y = causal_conv(u, w.float(), None, state, state_rows, off, qsl, seq_lens, silu=False)
+    q = y[:, :q_cols]
+    if temp_coef != 0.0:
+        q = q * (1.0 + temp_coef * torch.log(torch.floor((positions.float() + 1.0) / temp_every) + 1.0)).unsqueeze(1)
+    nk = num_kv_heads * dk
+    kv_write(cache, y[:, q_cols:q_cols + nk], y[:, q_cols + nk:], slot_mapping, koff, voff, num_kv_heads, dk, dv, block_size)
+    return q.to(x.dtype)
+
+
+# ----------------------------------------------------------------------------- attention in two maps
+DIFF_TARGET_GROUPS = 512  # workgroups that fill the 256 CUs two deep: steps of few rows split their keys up to this
+
+
+def differential_attention(q: torch.Tensor, cache: torch.Tensor, block_tables: torch.Tensor, qsl: torch.Tensor,
+                           seq_lens: torch.Tensor, koff: int, voff: int, num_heads: int, num_kv_heads: int, dk: int,
+                           dv: int, block_size: int, scale: float, softcap: float, lam: float, out_scale: float,
+                           eps: float, gate: Optional[torch.Tensor] = None, max_query_len: int = 0,
+                           max_seq_len: int = 0, num_singles: int = 0) -> torch.Tensor:
+    """Softmax attention in two maps over the same values, causal, through the paged cache (this step's keys
+    already written).  Query head h has two queries q [T, H, 2, dk]; a cached key row holds the two keys of a kv
+    head (K at `koff` as [G, BS, 2, dk], V at `voff` as [G, BS, dv]); head h reads kv head h // (H / G).
+        a_m = softmax over j <= i of cap(scale q_m . k_m,j), times the values        (m = 1, 2)
+        o = a_1 - lam a_2;   o <- o / sqrt(mean(o^2) + eps) * out_scale   over dv;   o <- o * sigmoid(gate)
+    with cap(s) = softcap tanh(s / softcap) (softcap <= 0: s itself) and gate [T, H*dv] (a row-strided view, optional).
+    Scores, weights, both maps' sums and the norm in fp32; returns [T, H*dv] in q's dtype.
+    num_singles: so many of the step's leading sequences have one row each (they run a form of their own when the
+    step also holds longer chunks); max_query_len / max_seq_len: host bounds on the chunks and contexts."""
+    T = q.shape[0]
+    if _gpu(q):
+        out = torch.empty(T, num_heads * dv, dtype=q.dtype, device=q.device)
+        S = seq_lens.numel()
+        bf = q.dtype == torch.bfloat16
+        mq = max(1, min(int(max_query_len) or T, T))
+        span = max(int(max_seq_len) or 16, 16)
+        # (first sequence, last sequence, its longest chunk): single tokens apart from chunks in a mixed step
+        spans = [(0, S, mq)] if mq == 1 or not 0 < num_singles < S or not bf else [(0, num_singles, 1), (num_singles, S, mq)]
+        for s0, s1, m in spans:
+            nsplit, part = 1, None
+            if bf:
+                tiles = (s1 - s0) * num_kv_heads * ext().differential_tiles(m, num_heads // num_kv_heads)
+                nsplit = max(1, min(32, DIFF_TARGET_GROUPS // max(tiles, 1), span // 128))
+                if nsplit > 1:
+                    part = torch.empty(T * num_heads * 2 * nsplit * (dv + 4), dtype=torch.float32, device=q.device)
+            ext().differential_attention(out, q, cache, block_tables[s0:s1], qsl[s0:s1 + 1], seq_lens[s0:s1], int(koff),
+                                         int(voff), num_heads, num_kv_heads, dk, dv, block_size, float(scale),
+                                         float(softcap), float(lam), float(out_scale), float(eps), gate, m, nsplit, part)
+        return out
+    out = torch.zeros(T, num_heads, dv, dtype=torch.float32)
+    G = num_kv_heads
+    kc = cache[:, koff:koff + G * block_size * 2 * dk].view(-1, G, block_size, 2, dk)
+    vc = cache[:, voff:voff + G * block_size * dv].view(-1, G, block_size, dv)
+    rep = num_heads // G
+    ql, sl = qsl.tolist(), seq_lens.tolist()
+    for s in range(len(sl)):
+        a, e = ql[s], ql[s + 1]
+        n = sl[s]
+        if e <= a:
+            continue
+        nb = -(-n // block_size)
+        blocks = block_tables[s, :nb].long()
+        K = kc[blocks].permute(0, 2, 1, 3, 4).reshape(nb * block_size, G, 2, dk)[:n].float().repeat_interleave(rep, dim=1)
+        V = vc[blocks].permute(0, 2, 1, 3).reshape(nb * block_size, G, dv)[:n].float().repeat_interleave(rep, dim=1)
+        sc = torch.einsum("ihmd,jhmd->hmij", q[a:e].reshape(e - a, num_heads, 2, dk).float(), K) * scale
+        if softcap > 0:
+            sc = softcap * torch.tanh(sc / softcap)
+        i = torch.arange(n - (e - a), n).unsqueeze(1)
+        sc = sc.masked_fill(torch.arange(n).unsqueeze(0) > i, float("-inf"))
+        am = torch.einsum("hmij,jhd->mihd", torch.softmax(sc, dim=-1), V)
+        out[a:e] = am[0] - lam * am[1]
+    y = (_rms(out, eps) * out_scale).reshape(T, num_heads * dv)
+    if gate is not None:
+        y = y * torch.sigmoid(gate.float())
+    return y.to(q.dtype)
+
+
 # ----------------------------------------------------------------------------- column scans
+def decay_lowrank(x: torch.Tensor, w: torch.Tensor, bias: torch.Tensor, tau: float) -> torch.Tensor:
+    """Logarithms of decays from a low-rank pair's inner values: log(sigmoid(w x + bias)) / tau, fp32 [T, N].
+    x [T, R] (row-strided view), w [N, R], bias [N]; products and sums in fp32."""
+    if _gpu(x):
+        out = torch.empty(x.shape[0], w.shape[0], dtype=torch.float32, device=x.device)
+        ext().decay_lowrank(out, x, w, bias, float(tau))
+        return out
+    return F.logsigmoid(F.linear(x.float(), w.float(), bias.float())) / tau
+
+
+def gla_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, loga: torch.Tensor, state: torch.Tensor,
+             state_rows: torch.Tensor, off: int, qsl: torch.Tensor, seq_lens: torch.Tensor, num_heads: int, dk: int,
+             dv: int, q_scale: float, max_query_len: int = 0) -> torch.Tensor:
+    """Gated linear attention with one decay per head and key channel:
+        S <- diag(exp(loga_t)) S + k_t v_t^T,   o_t = S^T (q_scale q_t)
+    so the read-out sees the token's own write.  q, k [T, H*dk], v [T, H*dv] (row-strided views), loga fp32
+    [T, H*dk] (<= 0).  Returns o fp32 [T, H*dv]; S (fp32, stored [H, dv, dk]) stays in the sequence's slot.
+    max_query_len: the step's longest chunk (host int); the step is a diagonal map of the state, so long chunks
+    are cut into pieces that run side by side (end states from an empty start, chained by the pieces' summed
+    logarithms, then the outputs)."""
+    T, H = q.shape[0], num_heads
+    if _gpu(q):
+        out = torch.empty(T, H * dv, dtype=torch.float32, device=q.device)
+        piece, npieces, loc, start = _scan_split(seq_lens.numel(), T, max_query_len, H * dv * dk, H, 4 * dv, q.device)
+        dec = torch.empty(seq_lens.numel() * npieces * H * dk, dtype=torch.float32, device=q.device) if npieces > 1 else None
+        ext().gla_scan(out, q, k, v, loga, state, state_rows, int(off), qsl, seq_lens, H, dk, dv, float(q_scale), piece,
+                       npieces, loc, start, dec, int(max_query_len))
+        return out
+    out = torch.zeros(T, H, dv, dtype=torch.float32)
+    qf, kf, vf = (q.float() * q_scale).reshape(T, H, dk), k.float().reshape(T, H, dk), v.float().reshape(T, H, dv)
+    a = torch.exp(loga).reshape(T, H, dk)
+    ql, sl, rows = qsl.tolist(), seq_lens.tolist(), state_rows.tolist()
+    for s in range(len(sl)):
+        b, e = ql[s], ql[s + 1]
+        if e <= b:
+            continue
+        S = state[rows[s], off:off + H * dv * dk].view(H, dv, dk)
+        if sl[s] - (e - b) == 0:
+            S.zero_()
+        for t in range(b, e):
+            S.mul_(a[t].unsqueeze(1)).add_(vf[t].unsqueeze(2) * kf[t].unsqueeze(1))
+            out[t] = (S * qf[t].unsqueeze(1)).sum(-1)
+    return out.reshape(T, H * dv)
+
+
 def ssd_scan(x: torch.Tensor, B: torch.Tensor, C: torch.Tensor, dt: torch.Tensor, dt_bias: torch.Tensor,
              A_log: torch.Tensor, D: torch.Tensor, state: torch.Tensor, state_rows: torch.Tensor, off: int,
              qsl: torch.Tensor, seq_lens: torch.Tensor, num_heads: int, groups: int, N: int, P: int,
@@ -773,22 +986,39 @@ def latent_attention(q: torch.Tensor, cache: torch.Tensor, block_tables: torch.T
 
 
 # ----------------------------------------------------------------------------- routed experts
-def route_topk(logits: torch.Tensor, k: int, renorm: bool = False, softmax: bool = False) -> tuple:
+def route_topk(logits: torch.Tensor, k: int, renorm: bool = False, softmax: bool = False, *,
+               correction: Optional[torch.Tensor] = None, groups: int = 1, keep: int = 1, scale: float = 1.0) -> tuple:
     """Router: scores = sigmoid(logits), or softmax over all experts (fp32 [T, E]); the k largest per
     token (ties: the lower index first), their scores as weights (renorm: divided by their sum).
+    The keyword forms: correction (fp32 [E]) is added to the scores for the choice only; with groups > 1 the experts
+    form that many equal runs of neighbours, a group's score is the sum of its two largest choice scores, and only
+    experts of the `keep` best groups can be chosen; weights are multiplied by scale.
     -> (weights fp32 [T, k], ids int32 [T, k])."""
     T, E = logits.shape
+    if E % groups or not 1 <= keep <= groups or k > keep * (E // groups):
+        raise ValueError(f"route_topk: {k} of {E} experts in {keep} of {groups} groups")
+    grouped = correction is not None or groups > 1 or scale != 1.0
     if _gpu(logits):
         w = torch.empty(T, k, dtype=torch.float32, device=logits.device)
         ids = torch.empty(T, k, dtype=torch.int32, device=logits.device)
-        ext().route_topk(w, ids, logits, bool(renorm), bool(softmax))
+        if grouped:
+            ext().route_grouped(w, ids, logits, correction, int(groups), int(keep), float(scale), bool(renorm), bool(softmax))
+        else:
+            ext().route_topk(w, ids, logits, bool(renorm), bool(softmax))
         return w, ids
     s = torch.softmax(logits.float(), dim=-1) if softmax else torch.sigmoid(logits.float())
-    order = torch.argsort(s, dim=-1, descending=True, stable=True)[:, :k]
+    c = s if correction is None else s + correction.float()
+    if groups > 1:
+        per = c.view(T, groups, E // groups)
+        gs = per.topk(min(2, E // groups), dim=-1)[0].sum(-1)
+        best = torch.argsort(gs, dim=-1, descending=True, stable=True)[:, :keep]
+        seen = torch.zeros(T, groups, dtype=torch.bool).scatter_(1, best, True)
+        c = per.masked_fill(~seen.unsqueeze(-1), float("-inf")).reshape(T, E)
+    order = torch.argsort(c, dim=-1, descending=True, stable=True)[:, :k]
     w = torch.gather(s, 1, order)
     if renorm:
-        w = w / w.sum(-1, keepdim=True)
-    return w, order.to(torch.int32)
+        w = w / (w.sum(-1, keepdim=True) + 1e-20)
+    return w * scale if scale != 1.0 else w, order.to(torch.int32)
 
 
 def capped_glu(gu: torch.Tensor, limit: float, alpha: float = 1.702) -> torch.Tensor:

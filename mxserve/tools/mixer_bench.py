@@ -375,7 +375,7 @@ def momuvik_rooflines(width: int, prompt: int, batch: int, context: int) -> list
         entry(f"rope_half_into/{mode}", t, 0.0, PEAK_F32, 4.0 * T * H * dr, f"{T} rows x {H} heads x {dr} turned entries")
         # routed experts: router, the two expert products with the capped activation, the sum
         f = RoutedExperts("f.", width, E, top, ff, 7.0)
-        w = {"f.router": rnd(E, width), "f._gu": rnd(E, 2 * ff, width) * width ** -0.5, "f._down": rnd(E, width, ff) * ff ** -0.5}
+        w = {"f.router": rnd(E, width), "f._in": rnd(E, width, 2 * ff) * width ** -0.5, "f._down": rnd(E, ff, width) * ff ** -0.5}
         h = rnd(T, width)
         t = _time(lambda: f.forward(h, w), 5)
         act = min(E, T * top)
@@ -466,7 +466,7 @@ def seradra_rooflines(width: int, prompt: int, batch: int, context: int) -> list
                   f"{T} rows x {H} heads x ~{int(kk)} keys of {ldk}+{rank}, bf16 MFMA peak")
         # routed experts: softmax scores on the outputs of plain SiLU units beside sigmoid scores on the inputs of capped ones
         h = rnd(T, width)
-        w = {"f.router": rnd(E, width), "f._gu": rnd(E, 2 * ff, width) * width ** -0.5, "f._down": rnd(E, width, ff) * ff ** -0.5}
+        w = {"f.router": rnd(E, width), "f._in": rnd(E, width, 2 * ff) * width ** -0.5, "f._down": rnd(E, ff, width) * ff ** -0.5}
         act = min(E, T * top)
         for name, f in (("routed_experts", RoutedExperts("f.", width, E, top, ff, None, score="softmax", weigh="output")),
                         ("routed_experts (momuvik)", RoutedExperts("f.", width, E, top, ff, 7.0))):
