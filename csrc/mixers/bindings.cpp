@@ -6,6 +6,7 @@
 #include <torch/extension.h>
 
 #include "column_scan.h"
+#include "differential_attention.h"
 
 namespace mxs {
 void launch_resid_update(float*, const void*, long, const void*, const void*, long, const void*, const void*, int,
@@ -44,7 +45,17 @@ void launch_causal_conv(void*, const void*, long, const void*, const void*, floa
                         const int*, int, int, int, int, int, bool, hipStream_t);
 void launch_gated_norm(void*, long, const float*, const void*, long, const void*, int, int, int, int, float, int, int,
                        float, bool, hipStream_t);
-bool launch_column_scan(const ScanArgs&, int, bool, bool, hipStream_t);
+bool launch_column_scan(const ScanArgs&, int, int, bool, hipStream_t);
+bool launch_decay_lowrank(float*, const void*, long, const void*, const void*, int, int, int, float, bool, hipStream_t);
+bool launch_streams(float*, int, const void*, long, const int64_t*, long, const void*, const void*, const float*, const void*,
+                    void*, int, int, float, float, bool, hipStream_t);
+void launch_act(void*, const void*, long, int, int, int, bool, bool, hipStream_t);
+void launch_conv_qkv_cache(void*, const void*, long, const void*, const void*, float*, long, const int*, long, const int*,
+                           const int*, int, int, const int64_t*, const int64_t*, void*, long, int, int, int, int, int, int,
+                           int, int, float, float, bool, bool, hipStream_t);
+int differential_tiles(int, int);
+bool launch_differential_attention(const DiffArgs&, int, int, bool, hipStream_t);
+bool launch_route_grouped(float*, int*, const float*, const float*, int, int, int, int, int, float, bool, bool, hipStream_t);
 bool launch_latent_attention(void*, float*, const void*, long, const void*, long, const int*, int, const int*, const int*,
                              int, int, int, int, int, int, int, float, int, const float*, int, bool, int, hipStream_t);
 void launch_latent_prep(void*, const void*, long, const void*, long, const int64_t*, const int64_t*, void*, long, int, int,
@@ -366,12 +377,12 @@ void gated_norm(at::Tensor out, at::Tensor o, at::Tensor gate, at::Tensor w, dou
                          gate_first ? 1 : 0, static_cast<float>(scale), bf, stream());
 }
 
-void column_scan(bool delta, at::Tensor out, at::Tensor q, at::Tensor k, at::Tensor v, at::Tensor beta, OptT a,
-                 at::Tensor dt_bias, at::Tensor A_log, OptT D, at::Tensor state, at::Tensor state_rows, int64_t off,
+void column_scan(int kind, at::Tensor out, at::Tensor q, at::Tensor k, at::Tensor v, OptT beta, OptT a,
+                 OptT dt_bias, OptT A_log, OptT D, at::Tensor state, at::Tensor state_rows, int64_t off,
                  at::Tensor qsl, at::Tensor seq_lens, int64_t H, int64_t G, int64_t dk, int64_t dv, double q_scale,
                  double unit_eps, int64_t piece = 1, int64_t npieces = 1, OptT sc_local = OptT(), OptT sc_start = OptT(),
                  OptT sc_decay = OptT(), int64_t mode = 0, int64_t max_q = 0) {
-  const bool bf = is_bf(q);
+  const bool bf = is_bf(q), delta = kind == mxs::kDeltaRule, gla = kind == mxs::kGatedLinear;
   const int64_t T = q.size(0), S = seq_lens.numel();
   TORCH_CHECK(G >= 1 && H % G == 0, "heads must divide over the q/k heads (groups)");
   mxs::ScanArgs p{};
@@ -383,18 +394,25 @@ void column_scan(bool delta, at::Tensor out, at::Tensor q, at::Tensor k, at::Ten
   p.k_stride = k.stride(0);
   p.v = mat(v, bf, T, H * dv, "v");
   p.v_stride = v.stride(0);
-  p.beta = mat(beta, bf, T, H, "beta");
-  p.beta_stride = beta.stride(0);
-  if (delta) {
-    TORCH_CHECK(a.has_value(), "the delta rule needs its decay pre-activations");
-    p.a = mat(*a, bf, T, H * dk, "a");
+  if (gla) {
+    TORCH_CHECK(a.has_value() && G == H, "gated linear attention: log decays, one q/k head per head");
+    p.a = mat(*a, false, T, H * dk, "log decays (fp32)");
     p.a_stride = a->stride(0);
   } else {
-    TORCH_CHECK(D.has_value(), "the state-space scan needs D");
+    TORCH_CHECK(beta.has_value() && dt_bias.has_value() && A_log.has_value(), "column scan: beta, dt_bias and A_log");
+    p.beta = mat(*beta, bf, T, H, "beta");
+    p.beta_stride = beta->stride(0);
+    if (delta) {
+      TORCH_CHECK(a.has_value(), "the delta rule needs its decay pre-activations");
+      p.a = mat(*a, bf, T, H * dk, "a");
+      p.a_stride = a->stride(0);
+    } else {
+      TORCH_CHECK(D.has_value(), "the state-space scan needs D");
+    }
+    p.dt_bias = f32n(dt_bias, delta ? H * dk : H, "dt_bias");
+    p.A_log = f32n(A_log, H, "A_log");
+    p.D = f32n(D, H, "D");
   }
-  p.dt_bias = f32n(OptT(dt_bias), delta ? H * dk : H, "dt_bias");
-  p.A_log = f32n(OptT(A_log), H, "A_log");
-  p.D = f32n(D, H, "D");
   p.state = f32(state, "state");
   TORCH_CHECK(state.dim() == 2 && off >= 0 && off + H * dk * dv <= state.size(1), "state slot too small for this layer");
   p.state_stride = state.stride(0);
@@ -412,11 +430,12 @@ void column_scan(bool delta, at::Tensor out, at::Tensor q, at::Tensor k, at::Ten
   p.piece = 1;
   p.npieces = 1;
   p.max_q = (max_q == 1 && T == S) ? 1 : 0;  // every sequence brings one row
-  if (npieces > 1) {  // pieces side by side: scratch [S, npieces, state] twice and [S, npieces, H]
+  if (npieces > 1) {  // pieces side by side: scratch [S, npieces, state] twice and the pieces' decays
     TORCH_CHECK(piece >= 16 && sc_local.has_value() && sc_start.has_value() && (delta || sc_decay.has_value()),
                 "a split scan needs its scratch pools");
     TORCH_CHECK(sc_local->numel() >= S * npieces * H * dk * (delta ? dv + dk : dv) &&
-                sc_start->numel() >= S * npieces * H * dk * dv && (delta || sc_decay->numel() >= S * npieces * H),
+                sc_start->numel() >= S * npieces * H * dk * dv &&
+                (delta || sc_decay->numel() >= S * npieces * H * (gla ? dk : 1)),
                 "scratch pools smaller than [S, npieces, state]");
     TORCH_CHECK(!delta || mode == 1 || mode == 2, "a split delta-rule scan is launched pass by pass");
     p.piece = static_cast<int>(piece);
@@ -426,14 +445,14 @@ void column_scan(bool delta, at::Tensor out, at::Tensor q, at::Tensor k, at::Ten
     p.sc_start = f32(*sc_start, "sc_start");
     p.sc_decay = delta ? nullptr : f32(*sc_decay, "sc_decay");
   }
-  TORCH_CHECK(mxs::launch_column_scan(p, static_cast<int>(S), delta, bf, stream()), "column scan: key / state size beyond 256");
+  TORCH_CHECK(mxs::launch_column_scan(p, static_cast<int>(S), kind, bf, stream()), "column scan: key / state size beyond 256");
 }
 
 void ssd_scan(at::Tensor out, at::Tensor x, at::Tensor B, at::Tensor C, at::Tensor dt, at::Tensor dt_bias, at::Tensor A_log,
               at::Tensor D, at::Tensor state, at::Tensor state_rows, int64_t off, at::Tensor qsl, at::Tensor seq_lens,
               int64_t H, int64_t G, int64_t N, int64_t P, int64_t piece, int64_t npieces, OptT sc_local, OptT sc_start,
               OptT sc_decay, int64_t max_q) {
-  column_scan(false, out, C, B, x, dt, OptT(), dt_bias, A_log, OptT(D), state, state_rows, off, qsl, seq_lens, H, G, N, P,
+  column_scan(mxs::kStateSpace, out, C, B, x, OptT(dt), OptT(), OptT(dt_bias), OptT(A_log), OptT(D), state, state_rows, off, qsl, seq_lens, H, G, N, P,
               1.0, 0.0, piece, npieces, sc_local, sc_start, sc_decay, 0, max_q);
 }
 
@@ -441,15 +460,170 @@ void delta_scan(at::Tensor out, at::Tensor q, at::Tensor k, at::Tensor v, at::Te
                 at::Tensor A_log, at::Tensor state, at::Tensor state_rows, int64_t off, at::Tensor qsl, at::Tensor seq_lens,
                 int64_t H, int64_t G, int64_t dk, int64_t dv, double q_scale, double unit_eps, int64_t mode, int64_t piece,
                 int64_t npieces, OptT sc_local, OptT sc_start, int64_t max_q) {
-  column_scan(true, out, q, k, v, beta, OptT(a), dt_bias, A_log, OptT(), state, state_rows, off, qsl, seq_lens, H, G, dk, dv,
+  column_scan(mxs::kDeltaRule, out, q, k, v, OptT(beta), OptT(a), OptT(dt_bias), OptT(A_log), OptT(), state, state_rows, off, qsl, seq_lens, H, G, dk, dv,
               q_scale, unit_eps, piece, npieces, sc_local, sc_start, OptT(), mode, max_q);
 }
+
+void gla_scan(at::Tensor out, at::Tensor q, at::Tensor k, at::Tensor v, at::Tensor loga, at::Tensor state,
+              at::Tensor state_rows, int64_t off, at::Tensor qsl, at::Tensor seq_lens, int64_t H, int64_t dk, int64_t dv,
+              double q_scale, int64_t piece, int64_t npieces, OptT sc_local, OptT sc_start, OptT sc_decay, int64_t max_q) {
+  column_scan(mxs::kGatedLinear, out, q, k, v, OptT(), OptT(loga), OptT(), OptT(), OptT(), state, state_rows, off, qsl, seq_lens,
+              H, H, dk, dv, q_scale, 0.0, piece, npieces, sc_local, sc_start, sc_decay, 0, max_q);
+}
+
+void decay_lowrank(at::Tensor out, at::Tensor x, at::Tensor w, at::Tensor bias, double tau) {
+  const bool bf = is_bf(x);
+  TORCH_CHECK(x.dim() == 2 && w.dim() == 2 && w.is_cuda() && w.is_contiguous() && is_bf(w) == bf && w.size(1) == x.size(1),
+              "decay_lowrank: x [T, R], w [N, R] of one dtype");
+  const int64_t T = x.size(0), N = w.size(0), R = w.size(1);
+  float* op = f32(out, "out");
+  TORCH_CHECK(out.dim() == 2 && out.size(0) == T && out.size(1) == N && tau != 0.0, "out: fp32 [T, N]; tau");
+  TORCH_CHECK(mxs::launch_decay_lowrank(op, mat(x, bf, T, R, "x"), x.stride(0), w.data_ptr(), vec(OptT(bias), bf, N, "bias"),
+                                        static_cast<int>(T), static_cast<int>(N), static_cast<int>(R), static_cast<float>(tau),
+                                        bf, stream()), "decay_lowrank: inner size beyond what the kernel holds");
+}
+
+// ---- several residual streams, activations (streams.hip)
+void streams_start(at::Tensor X, at::Tensor h, at::Tensor ids, at::Tensor table, at::Tensor w_in, at::Tensor norm_w, double eps,
+                   double w_offset) {
+  float* xp = f32(X, "X");
+  const bool bf = is_bf(table);
+  TORCH_CHECK(X.dim() == 3 && table.is_cuda() && table.dim() == 2 && table.is_contiguous() && table.size(1) == X.size(2),
+              "X [T, n, W], table [V, W]");
+  const int64_t T = X.size(0), n = X.size(1), W = X.size(2);
+  TORCH_CHECK(ids.is_cuda() && ids.scalar_type() == at::kLong && ids.is_contiguous() && ids.numel() == T, "ids: int64 [T]");
+  TORCH_CHECK(h.is_cuda() && h.is_contiguous() && h.dim() == 2 && h.size(0) == T && h.size(1) == W && is_bf(h) == bf, "h: [T, W]");
+  TORCH_CHECK(w_in.numel() == n, "w_in: [n]");
+  TORCH_CHECK(mxs::launch_streams(xp, static_cast<int>(n), table.data_ptr(), W, ids.data_ptr<int64_t>(), table.size(0), nullptr,
+                                  nullptr, f32(w_in, "w_in"), vec(OptT(norm_w), bf, W, "norm_w"), h.data_ptr(),
+                                  static_cast<int>(T), static_cast<int>(W), static_cast<float>(eps),
+                                  static_cast<float>(w_offset), bf, stream()), "more streams than the kernel holds (32)");
+}
+
+void streams_update(at::Tensor X, at::Tensor y, OptT bias, OptT scale, at::Tensor coeffs, at::Tensor norm_w, at::Tensor h,
+                    double eps, double w_offset) {
+  float* xp = f32(X, "X");
+  const bool bf = is_bf(y);
+  TORCH_CHECK(X.dim() == 3, "X [T, n, W]");
+  const int64_t T = X.size(0), n = X.size(1), W = X.size(2);
+  TORCH_CHECK(h.is_cuda() && h.is_contiguous() && h.dim() == 2 && h.size(0) == T && h.size(1) == W && is_bf(h) == bf, "h: [T, W]");
+  TORCH_CHECK(coeffs.numel() == n * n + 2 * n, "coeffs: [n * n + 2 n]");
+  TORCH_CHECK(mxs::launch_streams(xp, static_cast<int>(n), mat(y, bf, T, W, "y"), y.stride(0), nullptr, 0,
+                                  vec(bias, bf, W, "bias"), vec(scale, bf, W, "scale"), f32(coeffs, "coeffs"),
+                                  vec(OptT(norm_w), bf, W, "norm_w"), h.data_ptr(), static_cast<int>(T), static_cast<int>(W),
+                                  static_cast<float>(eps), static_cast<float>(w_offset), bf, stream()),
+              "more streams than the kernel holds (32)");
+}
+
+void act_any(at::Tensor out, at::Tensor x, int64_t kind, bool gated) {
+  const bool bf = is_bf(x);
+  TORCH_CHECK(kind >= 0 && kind <= 2, "unknown activation");
+  TORCH_CHECK(x.dim() == 2 && out.is_cuda() && out.is_contiguous() && out.dim() == 2 && out.size(0) == x.size(0) &&
+              out.size(1) * (gated ? 2 : 1) == x.size(1) && is_bf(out) == bf, "x [R, F] (gated: [R, 2F]), out [R, F]");
+  mxs::launch_act(out.data_ptr(), mat(x, bf, x.size(0), x.size(1), "x"), x.stride(0), static_cast<int>(x.size(0)),
+                  static_cast<int>(out.size(1)), static_cast<int>(kind), gated, bf, stream());
+}
+void unary_act(at::Tensor out, at::Tensor x, int64_t kind) { act_any(out, x, kind, false); }
+void act_mul(at::Tensor out, at::Tensor x, int64_t kind) { act_any(out, x, kind, true); }
 
 // ---- latent attention, routed experts (latent_experts.hip)
 const int64_t* i64c(const at::Tensor& t, int64_t n, const char* name) {
   TORCH_CHECK(t.is_cuda() && t.scalar_type() == at::kLong && t.is_contiguous() && t.numel() == n, name,
               ": expected ", n, " contiguous int64");
   return t.data_ptr<int64_t>();
+}
+
+// ---- convolved q/k/v and attention in two maps (rotary_conv.hip, differential_attention.hip)
+void conv_qkv_cache(at::Tensor q, at::Tensor x, at::Tensor w, OptT bias, at::Tensor state, at::Tensor state_rows, int64_t off,
+                    at::Tensor qsl, at::Tensor seq_lens, at::Tensor positions, at::Tensor slots, at::Tensor cache, int64_t koff,
+                    int64_t voff, int64_t G, int64_t dk, int64_t dv, int64_t bs, double temp_coef, double temp_every,
+                    int64_t max_q) {
+  const bool bf = is_bf(x);
+  TORCH_CHECK(x.dim() == 2 && w.dim() == 2 && w.is_cuda() && w.is_contiguous() && is_bf(w) == bf && w.size(1) == x.size(1),
+              "conv_qkv_cache: x [T, C], w [taps, C] of one dtype");
+  const int64_t T = x.size(0), C = x.size(1), taps = w.size(0), S = seq_lens.numel(), QC = C - G * (dk + dv);
+  TORCH_CHECK(taps >= 1 && QC >= 1 && q.is_cuda() && q.is_contiguous() && q.dim() == 2 && q.size(0) == T && q.size(1) == QC &&
+              is_bf(q) == bf, "q: contiguous [T, C - G (dk + dv)]");
+  TORCH_CHECK(temp_every != 0.0, "temp_every must not be zero");
+  check_cache(cache, bf, koff, voff, G, dk, dv, bs);
+  float* sp = f32(state, "state");
+  TORCH_CHECK(state.dim() == 2 && off >= 0 && off + (taps - 1) * C <= state.size(1), "state slot too small for this filter");
+  mxs::launch_conv_qkv_cache(q.data_ptr(), mat(x, bf, T, C, "x"), x.stride(0), w.data_ptr(), vec(bias, bf, C, "bias"), sp,
+                             state.stride(0), i32(state_rows, S, "state_rows"), off, i32(qsl, S + 1, "qsl"),
+                             i32(seq_lens, S, "seq_lens"), static_cast<int>(S), static_cast<int>(T),
+                             i64c(positions, T, "positions"), i64c(slots, T, "slot_mapping"), cache.data_ptr(),
+                             cache.stride(0), static_cast<int>(koff), static_cast<int>(voff), static_cast<int>(QC),
+                             static_cast<int>(G), static_cast<int>(dk), static_cast<int>(dv), static_cast<int>(bs),
+                             static_cast<int>(taps), static_cast<float>(temp_coef), static_cast<float>(temp_every),
+                             max_q == 1 && T == S, bf, stream());
+}
+
+int64_t differential_tiles(int64_t max_q, int64_t rep) {
+  return mxs::differential_tiles(static_cast<int>(max_q), static_cast<int>(rep));
+}
+
+void differential_attention(at::Tensor out, at::Tensor q, at::Tensor cache, at::Tensor block_tables, at::Tensor qsl,
+                            at::Tensor seq_lens, int64_t koff, int64_t voff, int64_t H, int64_t G, int64_t dk, int64_t dv,
+                            int64_t bs, double scale, double softcap, double lam, double out_scale, double eps, OptT gate,
+                            int64_t max_q, int64_t nsplit, OptT part) {
+  const bool bf = is_bf(q);
+  const int64_t T = q.size(0), S = seq_lens.numel();
+  check_cache(cache, bf, koff, voff, G, 2 * dk, dv, bs);
+  TORCH_CHECK(G >= 1 && H % G == 0 && dk >= 1 && dv >= 1, "query heads must divide over kv heads");
+  TORCH_CHECK(out.is_cuda() && out.is_contiguous() && out.dim() == 2 && out.size(0) == T && out.size(1) == H * dv &&
+              is_bf(out) == bf, "out: [T, H*dv]");
+  TORCH_CHECK(block_tables.is_cuda() && block_tables.scalar_type() == at::kInt && block_tables.dim() == 2 &&
+              block_tables.size(0) >= S && block_tables.size(1) >= 1 && block_tables.stride(1) == 1 &&
+              block_tables.stride(0) >= block_tables.size(1), "block_tables: int32 [S, max_blocks]");
+  mxs::DiffArgs a{};
+  a.out = out.data_ptr();
+  a.q = mat(q, bf, T, H * 2 * dk, "q");
+  a.q_stride = q.stride(0);
+  a.cache = cache.data_ptr();
+  a.block_stride = cache.stride(0);
+  a.block_tables = block_tables.data_ptr<int>();
+  a.bt_stride = static_cast<int>(block_tables.stride(0));
+  a.qsl = i32(qsl, S + 1, "qsl");
+  a.seq_lens = i32(seq_lens, S, "seq_lens");
+  a.n_rows = static_cast<int>(T);
+  a.koff = static_cast<int>(koff);
+  a.voff = static_cast<int>(voff);
+  a.H = static_cast<int>(H);
+  a.G = static_cast<int>(G);
+  a.dk = static_cast<int>(dk);
+  a.dv = static_cast<int>(dv);
+  a.max_q = static_cast<int>(std::max<int64_t>(1, std::min<int64_t>(max_q, T)));
+  a.scale = static_cast<float>(scale);
+  a.softcap = static_cast<float>(softcap);
+  a.lam = static_cast<float>(lam);
+  a.out_scale = static_cast<float>(out_scale);
+  a.eps = static_cast<float>(eps);
+  if (gate.has_value()) {
+    a.gate = mat(*gate, bf, T, H * dv, "gate");
+    a.gate_stride = gate->stride(0);
+  }
+  a.nsplit = 1;
+  if (nsplit > 1 && part.has_value()) {
+    TORCH_CHECK(part->numel() >= T * H * 2 * nsplit * (dv + 4), "part: fp32 [T, H, 2, nsplit, dv + 4]");
+    a.part = f32(*part, "part");
+    a.nsplit = static_cast<int>(nsplit);
+  }
+  TORCH_CHECK(mxs::launch_differential_attention(a, static_cast<int>(S), static_cast<int>(bs), bf, stream()),
+              "differential_attention: sizes beyond what the kernels hold (dv <= 512)");
+}
+
+void route_grouped(at::Tensor w, at::Tensor ids, at::Tensor logits, OptT correction, int64_t groups, int64_t keep, double scale,
+                   bool renorm, bool softmax) {
+  const float* lp = f32(logits, "logits");
+  TORCH_CHECK(logits.dim() == 2 && w.dim() == 2 && ids.dim() == 2, "logits [T, E], w / ids [T, k]");
+  const int64_t T = logits.size(0), E = logits.size(1), k = w.size(1);
+  TORCH_CHECK(groups >= 1 && E % groups == 0 && keep >= 1 && keep <= groups && k >= 1 && k <= keep * (E / groups) &&
+              w.size(0) == T && ids.size(0) == T && ids.size(1) == k, "k of E experts in the best groups; w, ids [T, k]");
+  TORCH_CHECK(ids.is_cuda() && ids.scalar_type() == at::kInt && ids.is_contiguous(), "ids: contiguous int32");
+  TORCH_CHECK(mxs::launch_route_grouped(f32(w, "w"), ids.data_ptr<int>(), lp, f32n(correction, E, "correction"),
+                                        static_cast<int>(T), static_cast<int>(E), static_cast<int>(k), static_cast<int>(groups),
+                                        static_cast<int>(keep), static_cast<float>(scale), renorm, softmax, stream()),
+              "route_grouped: more experts than the kernel holds");
 }
 
 void latent_prep(at::Tensor cq, at::Tensor dq, at::Tensor dkv, at::Tensor positions, at::Tensor slots, at::Tensor cache,
@@ -750,4 +924,14 @@ PYBIND11_MODULE(_M, m) {
   m.def("xielu", &xielu);
   m.def("qkv_prep_cache", &qkv_prep_cache);
   m.def("talking_attention", &talking_attention);
+  m.def("streams_start", &streams_start);
+  m.def("streams_update", &streams_update);
+  m.def("unary_act", &unary_act);
+  m.def("act_mul", &act_mul);
+  m.def("conv_qkv_cache", &conv_qkv_cache);
+  m.def("differential_tiles", &differential_tiles);
+  m.def("differential_attention", &differential_attention);
+  m.def("decay_lowrank", &decay_lowrank);
+  m.def("gla_scan", &gla_scan);
+  m.def("route_grouped", &route_grouped);
 }

@@ -1,5 +1,6 @@
 // Token-by-token recurrences whose state columns never interact (gfx950): the selective state space
-// with a scalar decay per head and token, and the gated delta rule with a decay per key channel.
+// with a scalar decay per head and token, the gated delta rule and gated linear attention with a decay
+// per key channel.
 //
 // The state S [dk, dv] of one (sequence, head) is stored transposed, [dv][dk], and split over
 // workgroups by 16 columns.  A column belongs to 16 neighbouring lanes (one DPP row); each keeps R
@@ -13,12 +14,13 @@
 // the previous 16 tokens' outputs are written while the next are staged.
 // Long chunks are cut into pieces that run side by side: pass 1 runs every piece from an empty state
 // and keeps its end state, and what carries a state across the piece (state space: the summed decay
-// exponents; delta rule: the piece's dk x dk transition matrix, from dk more columns started as the
+// exponents; gated linear attention: the summed logarithms per key channel; delta rule: the piece's dk x dk transition matrix, from dk more columns started as the
 // identity); the states at the pieces' starts are chained from those; pass 2 runs every piece again
 // from its true start and writes the outputs.
 // A token's sums run in an order fixed by the sizes alone, so cutting a prompt differently gives the
 // same bits.  State, decays, gates and every product are fp32; the operands come as bf16 or fp32.
 #include <algorithm>
+#include <type_traits>
 
 #include "mix_common.h"
 #include "column_scan.h"
@@ -96,24 +98,26 @@ template <int R> __device__ __forceinline__ void store_run(float* p, const float
 // token tid / 16; the run is the one whose rows it owns in the recurrence), one value element and the
 // token's scalar.  The loads of a stage are issued before the 16 tokens of the stage before it are
 // walked, so their latency hides behind that walk.
-template <int R, bool DELTA, int CG> struct StageRegs {
-  float k[R], q[R], a[DELTA ? R : 1], v[CG], b;
+template <int R, int KIND, int CG> struct StageRegs {
+  float k[R], q[R], a[KIND != kStateSpace ? R : 1], v[CG], b;
 };
 
-template <typename T, int R, bool DELTA, int CG>
-__device__ __forceinline__ void load_stage(StageRegs<R, DELTA, CG>& r, const ScanArgs& p, long row, bool ok, int kh, int hd,
+template <typename T, int R, int KIND, int CG>
+__device__ __forceinline__ void load_stage(StageRegs<R, KIND, CG>& r, const ScanArgs& p, long row, bool ok, int kh, int hd,
                                            int rp, int vcol, int flags) {
+  constexpr bool CH = KIND != kStateSpace;  // one decay per key channel
+  using A = typename std::conditional<KIND == kGatedLinear, float, T>::type;
   const T* qp = static_cast<const T*>(p.q);
   const T* kp = static_cast<const T*>(p.k);
   const T* vp = static_cast<const T*>(p.v);
   const T* bp = static_cast<const T*>(p.beta);
-  const T* ap = static_cast<const T*>(p.a);
+  const A* ap = static_cast<const A*>(p.a);
   const int d0 = rp * R;
 #pragma unroll
   for (int i = 0; i < R; ++i) {
     r.k[i] = 0.f;
     r.q[i] = 0.f;
-    if (DELTA) r.a[i] = 0.f;
+    if (CH) r.a[i] = 0.f;
   }
 #pragma unroll
   for (int j = 0; j < CG; ++j) r.v[j] = 0.f;
@@ -122,32 +126,33 @@ __device__ __forceinline__ void load_stage(StageRegs<R, DELTA, CG>& r, const Sca
   if (d0 + R <= p.dk) {
     load_run<R>(kp + row * p.k_stride + kh * p.dk + d0, r.k, flags & 1);
     load_run<R>(qp + row * p.q_stride + kh * p.dk + d0, r.q, flags & 2);
-    if (DELTA) load_run<R>(ap + row * p.a_stride + hd * p.dk + d0, r.a, flags & 4);
+    if constexpr (CH) load_run<R>(ap + row * p.a_stride + hd * p.dk + d0, r.a, flags & 4);
   } else {
 #pragma unroll
     for (int i = 0; i < R; ++i) {
       if (d0 + i < p.dk) {
         r.k[i] = ldf(kp + row * p.k_stride + kh * p.dk + d0 + i);
         r.q[i] = ldf(qp + row * p.q_stride + kh * p.dk + d0 + i);
-        if (DELTA) r.a[i] = ldf(ap + row * p.a_stride + hd * p.dk + d0 + i);
+        if constexpr (CH) r.a[i] = ldf(ap + row * p.a_stride + hd * p.dk + d0 + i);
       }
     }
   }
 #pragma unroll
   for (int j = 0; j < CG; ++j)
     if (vcol + j * kCols < p.dv) r.v[j] = ldf(vp + row * p.v_stride + hd * p.dv + vcol + j * kCols);
-  r.b = ldf(bp + row * p.beta_stride + hd);
+  if constexpr (KIND != kGatedLinear) r.b = ldf(bp + row * p.beta_stride + hd);
 }
 
 // ST: tokens per stage, 16, or 1 for steps of single tokens only.  CG: groups of 16 columns a workgroup
 // takes, each thread one column of every group: a step of single tokens is a read and a write of the
 // state and little else, so its workgroups take 64 columns and have four times the bytes in flight.
-template <typename T, int R, bool DELTA, int ST, int CG>
+template <typename T, int R, int KIND, int ST, int CG>
 __global__ void __launch_bounds__(256) column_scan_kernel(const ScanArgs p, int flags) {
   constexpr int DK = 16 * R;  // padded key size
+  constexpr bool DELTA = KIND == kDeltaRule, GLA = KIND == kGatedLinear, CH = DELTA || GLA;
   __shared__ __attribute__((aligned(16))) float sk[ST][DK];
   __shared__ __attribute__((aligned(16))) float sq[ST][DK];
-  __shared__ __attribute__((aligned(16))) float sg[DELTA ? ST : 1][DELTA ? DK : 4];
+  __shared__ __attribute__((aligned(16))) float sg[CH ? ST : 1][CH ? DK : 4];
   constexpr int WC = kCols * CG;  // columns per workgroup
   __shared__ float sv[ST][WC];
   __shared__ float so[ST][WC];
@@ -201,19 +206,24 @@ __global__ void __launch_bounds__(256) column_scan_kernel(const ScanArgs p, int 
       for (int i = 0; i < R; ++i) S[j][i] = rp * R + i == col - dv ? 1.f : 0.f;
     }
   }
-  float dsum = 0.f;  // state space, mode 1: this thread's share of the piece's summed decay exponents
-  const float eA = expf(p.A_log[hd]);
-  const float Dh = DELTA ? 0.f : p.D[hd];
+  // mode 1: this thread's share of the piece's summed decay exponents (gated linear: one sum per channel of its run)
+  float dsum[GLA ? R : 1];
+#pragma unroll
+  for (int i = 0; i < (GLA ? R : 1); ++i) dsum[i] = 0.f;
+  const float eA = GLA ? 0.f : expf(p.A_log[hd]);
+  const float Dh = CH ? 0.f : p.D[hd];
   float bias[DELTA ? R : 1];
-  if (DELTA) {
+  if (GLA) {
+    bias[0] = 0.f;
+  } else if (DELTA) {
 #pragma unroll
     for (int i = 0; i < R; ++i) bias[i] = rp * R + i < dk ? p.dt_bias[hd * dk + rp * R + i] : 0.f;
   } else {
     bias[0] = p.dt_bias[hd];
   }
   const int HV = H * dv;
-  StageRegs<R, DELTA, CG> rg;
-  load_stage<T, R, DELTA, CG>(rg, p, row0 + cl, cl < ST && cl < qlen, kh, hd, rp, c0 + rp, flags);
+  StageRegs<R, KIND, CG> rg;
+  load_stage<T, R, KIND, CG>(rg, p, row0 + cl, cl < ST && cl < qlen, kh, hd, rp, c0 + rp, flags);
   int prev_t0 = -1, prev_nt = 0;
   for (int t0 = 0; t0 < qlen; t0 += ST) {
     const int nt = min(ST, qlen - t0);
@@ -242,6 +252,15 @@ __global__ void __launch_bounds__(256) column_scan_kernel(const ScanArgs p, int 
         sg[cl][rp * R + i] = rp * R + i < dk ? expf(-eA * softplus_cs(rg.a[i] + bias[i])) : 0.f;
       }
       if (rp == 0) sb[cl] = sigmoid_f(rg.b);
+    } else if (GLA) {
+#pragma unroll
+      for (int i = 0; i < R; ++i) {
+        const float la = rg.a[CH ? i : 0];  // zero for rows past the chunk
+        sk[cl][rp * R + i] = rg.k[i];
+        sq[cl][rp * R + i] = rg.q[i] * p.q_scale;
+        sg[cl][rp * R + i] = rp * R + i < dk ? expf(la) : 0.f;
+        if (mode == 1) dsum[GLA ? i : 0] += la;
+      }
     } else {
 #pragma unroll
       for (int i = 0; i < R; ++i) {
@@ -252,7 +271,7 @@ __global__ void __launch_bounds__(256) column_scan_kernel(const ScanArgs p, int 
         const float dt = softplus_cs(rg.b + bias[0]);
         sb[cl] = dt;
         sa[cl] = expf(-eA * dt);
-        if (cl < nt) dsum += eA * dt;
+        if (cl < nt) dsum[0] += eA * dt;
       }
     }
     if (cl < ST) {
@@ -261,7 +280,7 @@ __global__ void __launch_bounds__(256) column_scan_kernel(const ScanArgs p, int 
     }
     __syncthreads();
     if (t0 + ST < qlen)  // the next stage's loads fly while this stage's tokens are walked
-      load_stage<T, R, DELTA, CG>(rg, p, row0 + t0 + ST + cl, cl < ST && t0 + ST + cl < qlen, kh, hd, rp, c0 + rp, flags);
+      load_stage<T, R, KIND, CG>(rg, p, row0 + t0 + ST + cl, cl < ST && t0 + ST + cl < qlen, kh, hd, rp, c0 + rp, flags);
     const bool readout = mode != 1;  // pass 1 wants a piece's end state only
     auto token = [&](int tt) {
       const float* kr = &sk[tt][rp * R];
@@ -296,6 +315,23 @@ __global__ void __launch_bounds__(256) column_scan_kernel(const ScanArgs p, int 
         } else {
 #pragma unroll
           for (int i = 0; i < R; ++i) Sj[i] += kr[i] * u;
+          o = 0.f;
+        }
+      } else if (GLA) {
+        const float* gr = &sg[tt][rp * R];
+        if (readout) {
+          float p0 = 0.f, p1 = 0.f;
+#pragma unroll
+          for (int i = 0; i < R; i += 2) {
+            Sj[i] = gr[i] * Sj[i] + vj * kr[i];
+            Sj[i + 1] = gr[i + 1] * Sj[i + 1] + vj * kr[i + 1];
+            p0 += Sj[i] * qr[i];
+            p1 += Sj[i + 1] * qr[i + 1];
+          }
+          o = row16_sum(p0 + p1);
+        } else {
+#pragma unroll
+          for (int i = 0; i < R; ++i) Sj[i] = gr[i] * Sj[i] + vj * kr[i];
           o = 0.f;
         }
       } else if (readout) {
@@ -334,8 +370,20 @@ __global__ void __launch_bounds__(256) column_scan_kernel(const ScanArgs p, int 
       if (c0 + j * kCols + rp < dv)
         p.out[static_cast<long>(row0 + prev_t0 + cl) * HV + hd * dv + c0 + j * kCols + rp] = so[cl][j * kCols + rp];
   }
-  if (!DELTA && mode == 1 && blockIdx.x == 0) {  // the piece's decay: exp(-sum) carries a state across it
-    if (rp == 0) sa[cl] = dsum;
+  if (GLA && mode == 1 && blockIdx.x == 0) {  // the piece's decays: exp(sum) carries a state across it, channel by channel
+    if (cl < ST) {
+#pragma unroll
+      for (int i = 0; i < R; ++i) sk[cl][rp * R + i] = dsum[GLA ? i : 0];
+    }
+    __syncthreads();
+    for (int d = tid; d < dk; d += blockDim.x) {
+      float t = 0.f;
+      for (int i = 0; i < ST; ++i) t += sk[i][d];
+      p.sc_decay[(static_cast<long>(s) * np + pc) * (static_cast<long>(H) * dk) + hd * dk + d] = t;
+    }
+  }
+  if (!CH && mode == 1 && blockIdx.x == 0) {  // the piece's decay: exp(-sum) carries a state across it
+    if (rp == 0) sa[cl] = dsum[0];
     __syncthreads();
     if (tid == 0) {
       float t = 0.f;
@@ -360,10 +408,10 @@ __global__ void __launch_bounds__(256) column_scan_kernel(const ScanArgs p, int 
   }
 }
 
-// Chains the pieces of a split state-space scan: sc_start[s][p] = the state at the start of piece p, from
+// Chains the pieces of a split diagonal scan (channel: the decays are summed logarithms per key channel): sc_start[s][p] = the state at the start of piece p, from
 // the slot (or zero for a sequence's first tokens), the pieces' end states from an empty state and
 // their decays.  One thread per state element, pieces walked in order.
-__global__ void __launch_bounds__(256) column_chain_kernel(const ScanArgs p) {
+__global__ void __launch_bounds__(256) column_chain_kernel(const ScanArgs p, int channel) {
   const int s = blockIdx.x, hd = blockIdx.y;
   const long per_head = static_cast<long>(p.dv) * p.dk;
   const long e = static_cast<long>(blockIdx.z) * 256 + threadIdx.x;
@@ -380,12 +428,15 @@ __global__ void __launch_bounds__(256) column_chain_kernel(const ScanArgs p) {
     const long sc = (static_cast<long>(s) * p.npieces + pc) * all + at;
     p.sc_start[sc] = cur;
     if (pc == np - 1) break;
-    cur = expf(-p.sc_decay[(static_cast<long>(s) * p.npieces + pc) * p.H + hd]) * cur + p.sc_local[sc];
+    const long piece = static_cast<long>(s) * p.npieces + pc;
+    const float a = channel ? p.sc_decay[piece * (static_cast<long>(p.H) * p.dk) + hd * p.dk + e % p.dk] : -p.sc_decay[piece * p.H + hd];
+    cur = expf(a) * cur + p.sc_local[sc];
   }
 }
 
-template <typename T, bool DELTA>
+template <typename T, int KIND>
 static bool launch_cs(const ScanArgs& a, int S, hipStream_t st) {
+  constexpr bool DELTA = KIND == kDeltaRule;
   const int ncols = (DELTA && a.mode == 1) ? a.dv + a.dk : a.dv;
   const int wc = a.max_q == 1 ? 4 * kCols : kCols;  // columns per workgroup
   const dim3 grid((ncols + wc - 1) / wc, a.H, S * a.npieces), block(256);
@@ -393,17 +444,20 @@ static bool launch_cs(const ScanArgs& a, int S, hipStream_t st) {
   const int R = a.dk <= 32 ? 2 : a.dk <= 64 ? 4 : a.dk <= 128 ? 8 : 16;
   // which operands' runs of R elements are aligned to their size (16 bytes at most): 1 k, 2 q, 4 a, 8 state
   const size_t es = sizeof(T), al = std::min<size_t>(16, R * es), sal = std::min<size_t>(16, R * 4);
-  auto ok = [&](const void* ptr, long stride) {
-    return ptr != nullptr && reinterpret_cast<uintptr_t>(ptr) % al == 0 && (stride * es) % al == 0 && (a.dk * es) % al == 0;
+  auto fits = [&](const void* ptr, long stride, size_t e, size_t n) {
+    return ptr != nullptr && reinterpret_cast<uintptr_t>(ptr) % n == 0 && (stride * e) % n == 0 && (a.dk * e) % n == 0;
   };
-  int flags = (ok(a.k, a.k_stride) ? 1 : 0) | (ok(a.q, a.q_stride) ? 2 : 0) | (DELTA && ok(a.a, a.a_stride) ? 4 : 0);
+  auto ok = [&](const void* ptr, long stride) { return fits(ptr, stride, es, al); };
+  int flags = (ok(a.k, a.k_stride) ? 1 : 0) | (ok(a.q, a.q_stride) ? 2 : 0);
+  if (DELTA && ok(a.a, a.a_stride)) flags |= 4;
+  if (KIND == kGatedLinear && fits(a.a, a.a_stride, sizeof(float), sal)) flags |= 4;
   if (reinterpret_cast<uintptr_t>(a.state) % sal == 0 && (a.state_stride * 4) % sal == 0 && (a.off * 4) % sal == 0 &&
       (a.dk * 4) % sal == 0)
     flags |= 8;
 #define MIX_CS(R)                                                                                              \
   do {                                                                                                         \
-    if (a.max_q == 1) hipLaunchKernelGGL((column_scan_kernel<T, R, DELTA, 1, 4>), grid, block, 0, st, a, flags);  \
-    else hipLaunchKernelGGL((column_scan_kernel<T, R, DELTA, kST, 1>), grid, block, 0, st, a, flags);             \
+    if (a.max_q == 1) hipLaunchKernelGGL((column_scan_kernel<T, R, KIND, 1, 4>), grid, block, 0, st, a, flags);  \
+    else hipLaunchKernelGGL((column_scan_kernel<T, R, KIND, kST, 1>), grid, block, 0, st, a, flags);             \
   } while (0)
   if (a.dk <= 32) MIX_CS(2);
   else if (a.dk <= 64) MIX_CS(4);
@@ -415,30 +469,80 @@ static bool launch_cs(const ScanArgs& a, int S, hipStream_t st) {
   return true;
 }
 
-static bool launch_pass(const ScanArgs& a, int S, bool delta, bool bf, hipStream_t st) {
-  if (bf) return delta ? launch_cs<bf16_t, true>(a, S, st) : launch_cs<bf16_t, false>(a, S, st);
-  return delta ? launch_cs<float, true>(a, S, st) : launch_cs<float, false>(a, S, st);
+static bool launch_pass(const ScanArgs& a, int S, int kind, bool bf, hipStream_t st) {
+  if (kind == kDeltaRule) return bf ? launch_cs<bf16_t, kDeltaRule>(a, S, st) : launch_cs<float, kDeltaRule>(a, S, st);
+  if (kind == kGatedLinear) return bf ? launch_cs<bf16_t, kGatedLinear>(a, S, st) : launch_cs<float, kGatedLinear>(a, S, st);
+  return bf ? launch_cs<bf16_t, kStateSpace>(a, S, st) : launch_cs<float, kStateSpace>(a, S, st);
 }
 
-bool launch_column_scan(const ScanArgs& a0, int S, bool delta, bool bf, hipStream_t st) {
+bool launch_column_scan(const ScanArgs& a0, int S, int kind, bool bf, hipStream_t st) {
   if (S == 0 || a0.n_rows == 0) return true;
   ScanArgs a = a0;
   if (a.npieces <= 1) {
     a.mode = 0;
     a.piece = 1;
     a.npieces = 1;
-    return launch_pass(a, S, delta, bf, st);
+    return launch_pass(a, S, kind, bf, st);
   }
   // the delta rule's step is no diagonal map of the state: the caller runs its passes one by one and
   // chains the pieces with matrix products in between (mxserve/ops/seqmix.py delta_scan)
-  if (delta) return (a.mode == 1 || a.mode == 2) && launch_pass(a, S, true, bf, st);
+  if (kind == kDeltaRule) return (a.mode == 1 || a.mode == 2) && launch_pass(a, S, kind, bf, st);
   a.mode = 1;
-  if (!launch_pass(a, S, false, bf, st)) return false;
+  if (!launch_pass(a, S, kind, bf, st)) return false;
   const long per_head = static_cast<long>(a.dv) * a.dk;
-  hipLaunchKernelGGL(column_chain_kernel, dim3(S, a.H, static_cast<unsigned>((per_head + 255) / 256)), dim3(256), 0, st, a);
+  hipLaunchKernelGGL(column_chain_kernel, dim3(S, a.H, static_cast<unsigned>((per_head + 255) / 256)), dim3(256), 0, st, a,
+                     kind == kGatedLinear ? 1 : 0);
   MXS_CHECK_LAUNCH();
   a.mode = 2;
-  return launch_pass(a, S, false, bf, st);
+  return launch_pass(a, S, kind, bf, st);
+}
+
+// Logarithms of decays from a low-rank pair: out[t, n] = log(sigmoid(x[t] . w[n] + bias[n])) / tau.  A workgroup
+// takes 16 tokens (their inner values in LDS) and 256 columns, a thread one column.
+constexpr int kDecayTokens = 16;
+template <typename T>
+__global__ void __launch_bounds__(256) decay_lowrank_kernel(float* __restrict__ out, const T* __restrict__ x, long x_stride,
+                                                            const T* __restrict__ w, const T* __restrict__ bias, int rows,
+                                                            int N, int R, float inv_tau) {
+  extern __shared__ float xl[];  // [kDecayTokens][R]
+  const int t0 = blockIdx.x * kDecayTokens, nt = min(kDecayTokens, rows - t0);
+  for (int i = threadIdx.x; i < nt * R; i += 256) {
+    const int t = i / R;
+    xl[i] = ldf(x + static_cast<long>(t0 + t) * x_stride + (i - t * R));
+  }
+  __syncthreads();
+  const int n = blockIdx.y * 256 + threadIdx.x;
+  if (n >= N) return;
+  const T* wr = w + static_cast<long>(n) * R;
+  float acc[kDecayTokens];
+  const float b = ldf(bias + n);
+#pragma unroll
+  for (int t = 0; t < kDecayTokens; ++t) acc[t] = b;
+  for (int r = 0; r < R; ++r) {
+    const float wv = ldf(wr + r);
+#pragma unroll
+    for (int t = 0; t < kDecayTokens; ++t)
+      if (t < nt) acc[t] += wv * xl[t * R + r];
+  }
+#pragma unroll
+  for (int t = 0; t < kDecayTokens; ++t)
+    if (t < nt) out[static_cast<long>(t0 + t) * N + n] = logsigmoid_f(acc[t]) * inv_tau;
+}
+
+bool launch_decay_lowrank(float* out, const void* x, long x_stride, const void* w, const void* bias, int rows, int N, int R,
+                          float tau, bool bf, hipStream_t st) {
+  if (rows == 0 || N == 0) return true;
+  const size_t shm = static_cast<size_t>(kDecayTokens) * R * sizeof(float);
+  if (shm > 60 * 1024) return false;
+  const dim3 grid((rows + kDecayTokens - 1) / kDecayTokens, (N + 255) / 256);
+  if (bf)
+    hipLaunchKernelGGL(decay_lowrank_kernel<bf16_t>, grid, dim3(256), shm, st, out, (const bf16_t*)x, x_stride, (const bf16_t*)w,
+                       (const bf16_t*)bias, rows, N, R, 1.f / tau);
+  else
+    hipLaunchKernelGGL(decay_lowrank_kernel<float>, grid, dim3(256), shm, st, out, (const float*)x, x_stride, (const float*)w,
+                       (const float*)bias, rows, N, R, 1.f / tau);
+  MXS_CHECK_LAUNCH();
+  return true;
 }
 
 }  // namespace mxs

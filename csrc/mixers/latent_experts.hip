@@ -6,6 +6,8 @@
 //                   rotary turn (half-split or neighbouring pairs) of the shared key part, both written into the token's page row
 //   rope_half_into  per token and head: the rotated part of the query into its columns of the folded query
 //   route_topk      sigmoid or softmax scores, the k largest per token (a wave per token)
+//   route_grouped   the same with a correction on the scores for the choice, experts limited to the best groups of
+//                   neighbours, and scaled weights
 //   capped_glu      g = min(gate, L), u = clamp(up, -L, L), g * sigmoid(alpha g) * (u + 1)
 //   expert_align    counting sort of the (token, slot) pairs by expert: offsets and each pair's sorted row
 //   gather_scaled   sorted rows = routing weight * the token's input
@@ -122,6 +124,83 @@ __global__ void __launch_bounds__(256) route_topk_kernel(float* __restrict__ w, 
   if (renorm && lane == 0) {
     const float inv = 1.f / total;
     for (int j = 0; j < k; ++j) w[static_cast<long>(t) * k + j] *= inv;  // own writes
+  }
+}
+
+// A wave per token.  The wave's choice scores (score + correction) wait in LDS [E]; lanes own groups first (the
+// sum of a group's two largest), `keep` passes of a wave-wide arg-max open the best groups and the others'
+// choice scores become -inf, then k passes pick the experts (ties: the lower index), each taken one
+// becoming -inf too.  The weights are the plain scores, read again from the logits.
+__global__ void __launch_bounds__(256) route_grouped_kernel(float* __restrict__ w, int* __restrict__ ids,
+                                                            const float* __restrict__ logits,
+                                                            const float* __restrict__ correction, int T, int E, int k,
+                                                            int groups, int keep, float scale, int renorm, int softmax) {
+  extern __shared__ float lds[];
+  const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
+  const int t = blockIdx.x * (blockDim.x >> 6) + wid;
+  if (t >= T) return;  // wave-uniform; no workgroup barrier below
+  const int per = E / groups;
+  float* c = lds + wid * (E + groups);  // [E] choice scores, then [groups] group scores
+  float* gs = c + E;
+  const float* z = logits + static_cast<long>(t) * E;
+  float zmax = 0.f, zinv = 1.f;
+  if (softmax) {
+    float mx = -INFINITY;
+    for (int e = lane; e < E; e += 64) mx = fmaxf(mx, z[e]);
+    zmax = wave_max(mx);
+    float sm = 0.f;
+    for (int e = lane; e < E; e += 64) sm += expf(z[e] - zmax);
+    zinv = 1.f / wave_sum(sm);
+  }
+  auto score = [&](int e) { return softmax ? expf(z[e] - zmax) * zinv : sigmoid_f(z[e]); };
+  for (int e = lane; e < E; e += 64) c[e] = score(e) + (correction ? correction[e] : 0.f);
+  // the best of v[0 .. n), lower index first among equals, the same in every lane; it becomes -inf
+  auto take = [&](float* v, int n) {
+    wave_sync();
+    float best = -INFINITY;
+    int bi = 0x7fffffff;
+    for (int e = lane; e < n; e += 64)
+      if (v[e] > best) { best = v[e]; bi = e; }
+#pragma unroll
+    for (int o = 32; o > 0; o >>= 1) {
+      const float ob = __shfl_xor(best, o, 64);
+      const int oi = __shfl_xor(bi, o, 64);
+      if (ob > best || (ob == best && oi < bi)) { best = ob; bi = oi; }
+    }
+    wave_sync();
+    if (bi < n && (bi & 63) == lane) v[bi] = -INFINITY;
+    return bi;
+  };
+  if (groups > 1 && keep < groups) {
+    wave_sync();
+    for (int g = lane; g < groups; g += 64) {
+      float a = -INFINITY, b = -INFINITY;  // the two largest
+      for (int e = g * per; e < (g + 1) * per; ++e) {
+        const float v = c[e];
+        if (v > a) { b = a; a = v; }
+        else if (v > b) b = v;
+      }
+      gs[g] = per > 1 ? a + b : a;
+    }
+    for (int j = 0; j < keep; ++j) take(gs, groups);  // an open group's score is now -inf
+    wave_sync();
+    for (int e = lane; e < E; e += 64)
+      if (gs[e / per] != -INFINITY) c[e] = -INFINITY;
+  }
+  float total = 0.f;
+  for (int j = 0; j < k; ++j) {
+    int bi = take(c, E);
+    if (bi >= E) bi = 0;  // no finite choice score left (NaN logits): stay inside the table
+    const float sc = score(bi);
+    total += sc;
+    if (lane == 0) {
+      w[static_cast<long>(t) * k + j] = renorm ? sc : sc * scale;
+      ids[static_cast<long>(t) * k + j] = bi;
+    }
+  }
+  if (renorm && lane == 0) {
+    const float den = total + 1e-20f;
+    for (int j = 0; j < k; ++j) w[static_cast<long>(t) * k + j] = w[static_cast<long>(t) * k + j] / den * scale;  // own writes
   }
 }
 
@@ -253,6 +332,17 @@ void launch_route_topk(float* w, int* ids, const float* logits, int T, int E, in
   hipLaunchKernelGGL(route_topk_kernel, dim3((T + 3) / 4), dim3(256), 0, st, w, ids, logits, T, E, k, renorm ? 1 : 0,
                      softmax ? 1 : 0);
   MXS_CHECK_LAUNCH();
+}
+
+bool launch_route_grouped(float* w, int* ids, const float* logits, const float* correction, int T, int E, int k, int groups,
+                          int keep, float scale, bool renorm, bool softmax, hipStream_t st) {
+  if (T == 0) return true;
+  const size_t shm = 4 * static_cast<size_t>(E + groups) * sizeof(float);
+  if (shm > 60 * 1024) return false;
+  hipLaunchKernelGGL(route_grouped_kernel, dim3((T + 3) / 4), dim3(256), shm, st, w, ids, logits, correction, T, E, k, groups,
+                     keep, scale, renorm ? 1 : 0, softmax ? 1 : 0);
+  MXS_CHECK_LAUNCH();
+  return true;
 }
 
 void launch_capped_glu(void* out, const void* gu, long gu_stride, int rows, int F, float limit, float alpha, bool bf,

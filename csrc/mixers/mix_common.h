@@ -66,6 +66,13 @@ __device__ __forceinline__ float silu_f(float z) { return z / (1.f + expf(-z)); 
 __device__ __forceinline__ float sigmoid_f(float z) { return 1.f / (1.f + expf(-z)); }
 __device__ __forceinline__ float logsigmoid_f(float z) { return z < 0.f ? z - log1pf(expf(z)) : -log1pf(expf(-z)); }
 
+// LDS written by some lanes of a wave is read by others of the same wave after this
+__device__ __forceinline__ void wave_sync() {
+  __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
+  __builtin_amdgcn_wave_barrier();
+  __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
+}
+
 // sequence of flattened row t: the last s with qsl[s] <= t
 __device__ __forceinline__ int seq_of_row(const int* __restrict__ qsl, int S, int t) {
   int lo = 0, hi = S - 1;

@@ -1,7 +1,7 @@
 // Kernels around rotary attention, short causal convolutions and gated output norms (gfx950):
 // scaled embedding rows into the fp32 stream, SiLU(gate) * up, q/k head norm + rotary pairs + paged
 // cache write in one launch, turning attention outputs back, the convolution with its carried
-// inputs, and the norm of a recurrent mixer's read-out with its gate.  Activations and weights are
+// inputs (alone, or with the query factor and the page write), and the norm of a recurrent mixer's read-out with its gate.  Activations and weights are
 // bf16 or fp32; angles, norms, sums and activations are fp32 with one rounding at the store.
 #include "mix_common.h"
 
@@ -195,11 +195,93 @@ __global__ void __launch_bounds__(256) causal_conv_kernel(T* __restrict__ out, c
   else stf(out + static_cast<long>(t) * C + c, acc[0]);
 }
 
-// The state after the step: the last taps-1 inputs of (old state ++ chunk).  Row r of the new state
+// The convolution without activation, from the fused projection to what attention reads: u = x + bias, the
+// filter over u, query columns (the first QC) times a factor that grows with the position, keys and values
+// (per kv head dk and dv columns) into the token's page rows.  A thread takes V consecutive channels as above
+// (WIDE: no piece crosses from one head to the next).  single: every sequence brings one row, and the thread
+// that filtered its channels also replaces the carried inputs.
+template <typename T, bool WIDE>
+__global__ void __launch_bounds__(256) conv_qkv_cache_kernel(
+    T* __restrict__ q, const T* __restrict__ x, long x_stride, const T* __restrict__ w, const T* __restrict__ bias,
+    float* __restrict__ state, long state_stride, const int* __restrict__ state_rows, long off, const int* __restrict__ qsl,
+    const int* __restrict__ seq_lens, int S, const int64_t* __restrict__ positions, const int64_t* __restrict__ slots,
+    T* __restrict__ cache, long block_stride, int koff, int voff, int QC, int G, int dk, int dv, int bs, int taps,
+    float temp_coef, float temp_every, int single) {
+  constexpr int V = WIDE ? Piece<T>::N : 1;
+  const int C = QC + G * (dk + dv);
+  const int t = blockIdx.x;
+  const int c = (blockIdx.y * 256 + threadIdx.x) * V;
+  if (c >= C) return;
+  const int s = single ? t : seq_of_row(qsl, S, t);
+  const int row0 = qsl[s], qlen = qsl[s + 1] - row0;
+  const int i = t - row0;
+  const bool fresh = seq_lens[s] - qlen <= 0;
+  float* st = state + static_cast<long>(state_rows[s]) * state_stride + off;
+  float acc[V], xv[V], wv[V], bv[V];
+#pragma unroll
+  for (int e = 0; e < V; ++e) acc[e] = bv[e] = 0.f;
+  if (bias) {
+    if constexpr (WIDE) load_piece(bias + c, bv);
+    else bv[0] = ldf(bias + c);
+  }
+  for (int j = 0; j < taps; ++j) {
+    const int src = i - (taps - 1 - j);
+    if (src < 0 && fresh) continue;
+    if constexpr (WIDE) {
+      if (src >= 0) {
+        load_piece(x + static_cast<long>(row0 + src) * x_stride + c, xv);
+#pragma unroll
+        for (int e = 0; e < V; ++e) xv[e] += bv[e];
+      } else {
+        const float* sp = st + static_cast<long>(taps - 1 + src) * C + c;
+#pragma unroll
+        for (int e = 0; e < V; e += 4) load_piece(sp + e, xv + e);
+      }
+      load_piece(w + static_cast<long>(j) * C + c, wv);
+    } else {
+      xv[0] = src >= 0 ? ldf(x + static_cast<long>(row0 + src) * x_stride + c) + bv[0]
+                       : st[static_cast<long>(taps - 1 + src) * C + c];
+      wv[0] = ldf(w + static_cast<long>(j) * C + c);
+    }
+#pragma unroll
+    for (int e = 0; e < V; ++e) acc[e] += wv[e] * xv[e];
+  }
+  if (single && taps > 1) {  // xv holds this row's u (the last tap): the carried inputs move up by one
+    for (int r = 0; r < taps - 1; ++r) {
+#pragma unroll
+      for (int e = 0; e < V; ++e) {
+        const float nv = r == taps - 2 ? xv[e] : (fresh ? 0.f : st[static_cast<long>(r + 1) * C + c + e]);
+        st[static_cast<long>(r) * C + c + e] = nv;
+      }
+    }
+  }
+  T* dst;
+  if (c < QC) {
+    if (temp_coef != 0.f) {
+      const float f = 1.f + temp_coef * logf(floorf((static_cast<float>(positions[t]) + 1.f) / temp_every) + 1.f);
+#pragma unroll
+      for (int e = 0; e < V; ++e) acc[e] *= f;
+    }
+    dst = q + static_cast<long>(t) * QC + c;
+  } else {
+    const int64_t slot = slots[t];
+    if (slot < 0) return;
+    const int nk = G * dk;
+    const bool key = c < QC + nk;
+    const int cc = key ? c - QC : c - QC - nk, d = key ? dk : dv;
+    const int g = cc / d;
+    dst = cache + (slot / bs) * block_stride + (key ? koff : voff) + (static_cast<long>(g) * bs + slot % bs) * d + (cc - g * d);
+  }
+  if constexpr (WIDE) store_piece(dst, acc);
+  else stf(dst, acc[0]);
+}
+
+// The state after the step: the last taps-1 inputs (plus bias) of (old state ++ chunk).  Row r of the new state
 // reads old row r + n or a chunk row, so one thread per channel walking r upwards never reads what it
 // has already replaced.  Runs after causal_conv_kernel on the same stream.
 template <typename T>
-__global__ void __launch_bounds__(256) conv_state_kernel(const T* __restrict__ x, long x_stride, float* __restrict__ state,
+__global__ void __launch_bounds__(256) conv_state_kernel(const T* __restrict__ x, long x_stride, const T* __restrict__ bias,
+                                                         float* __restrict__ state,
                                                          long state_stride, const int* __restrict__ state_rows, long off,
                                                          const int* __restrict__ qsl, const int* __restrict__ seq_lens,
                                                          int n_rows, int C, int taps) {
@@ -212,10 +294,11 @@ __global__ void __launch_bounds__(256) conv_state_kernel(const T* __restrict__ x
   if (n <= 0) return;
   const bool fresh = seq_lens[s] - n <= 0;
   float* st = state + static_cast<long>(state_rows[s]) * state_stride + off;
+  const float b = bias ? ldf(bias + c) : 0.f;
   for (int r = 0; r < taps - 1; ++r) {
     const int src = n - (taps - 1) + r;
     float xv = 0.f;
-    if (src >= 0) xv = ldf(x + static_cast<long>(row0 + src) * x_stride + c);
+    if (src >= 0) xv = ldf(x + static_cast<long>(row0 + src) * x_stride + c) + b;
     else if (!fresh) xv = st[static_cast<long>(taps - 1 + src) * C + c];
     st[static_cast<long>(r) * C + c] = xv;
   }
@@ -330,8 +413,39 @@ void launch_causal_conv(void* out, const void* x, long x_stride, const void* w, 
   }
   MXS_CHECK_LAUNCH();
   if (taps > 1) {
-    MIX_DISPATCH(bf, hipLaunchKernelGGL(conv_state_kernel<T>, dim3(S, cb), dim3(256), 0, st, (const T*)x, x_stride, state,
-                                        state_stride, state_rows, off, qsl, seq_lens, rows, C, taps));
+    MIX_DISPATCH(bf, hipLaunchKernelGGL(conv_state_kernel<T>, dim3(S, cb), dim3(256), 0, st, (const T*)x, x_stride,
+                                        (const T*)nullptr, state, state_stride, state_rows, off, qsl, seq_lens, rows, C, taps));
+    MXS_CHECK_LAUNCH();
+  }
+}
+
+void launch_conv_qkv_cache(void* q, const void* x, long x_stride, const void* w, const void* bias, float* state,
+                           long state_stride, const int* state_rows, long off, const int* qsl, const int* seq_lens, int S,
+                           int rows, const int64_t* positions, const int64_t* slots, void* cache, long block_stride, int koff,
+                           int voff, int QC, int G, int dk, int dv, int bs, int taps, float temp_coef, float temp_every,
+                           bool single, bool bf, hipStream_t st) {
+  if (rows == 0 || S == 0) return;
+  const int C = QC + G * (dk + dv), v = bf ? 8 : 4;
+  auto al = [](const void* ptr) { return reinterpret_cast<uintptr_t>(ptr) % 16 == 0; };
+  const bool wide = QC % v == 0 && dk % v == 0 && dv % v == 0 && x_stride % v == 0 && koff % v == 0 && voff % v == 0 &&
+                    block_stride % v == 0 && al(x) && al(w) && al(q) && al(cache) && (bias == nullptr || al(bias)) &&
+                    al(state) && state_stride % 4 == 0 && off % 4 == 0;
+  const dim3 grid(rows, ((wide ? C / v : C) + 255) / 256);
+  if (wide) {
+    MIX_DISPATCH(bf, hipLaunchKernelGGL((conv_qkv_cache_kernel<T, true>), grid, dim3(256), 0, st, (T*)q, (const T*)x, x_stride,
+                                        (const T*)w, (const T*)bias, state, state_stride, state_rows, off, qsl, seq_lens, S,
+                                        positions, slots, (T*)cache, block_stride, koff, voff, QC, G, dk, dv, bs, taps,
+                                        temp_coef, temp_every, single ? 1 : 0));
+  } else {
+    MIX_DISPATCH(bf, hipLaunchKernelGGL((conv_qkv_cache_kernel<T, false>), grid, dim3(256), 0, st, (T*)q, (const T*)x, x_stride,
+                                        (const T*)w, (const T*)bias, state, state_stride, state_rows, off, qsl, seq_lens, S,
+                                        positions, slots, (T*)cache, block_stride, koff, voff, QC, G, dk, dv, bs, taps,
+                                        temp_coef, temp_every, single ? 1 : 0));
+  }
+  MXS_CHECK_LAUNCH();
+  if (taps > 1 && !single) {
+    MIX_DISPATCH(bf, hipLaunchKernelGGL(conv_state_kernel<T>, dim3(S, (C + 255) / 256), dim3(256), 0, st, (const T*)x, x_stride,
+                                        (const T*)bias, state, state_stride, state_rows, off, qsl, seq_lens, rows, C, taps));
     MXS_CHECK_LAUNCH();
   }
 }
