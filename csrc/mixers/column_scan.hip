@@ -498,31 +498,44 @@ bool launch_column_scan(const ScanArgs& a0, int S, int kind, bool bf, hipStream_
 }
 
 // Logarithms of decays from a low-rank pair: out[t, n] = log(sigmoid(x[t] . w[n] + bias[n])) / tau.  A workgroup
-// takes 16 tokens (their inner values in LDS) and 256 columns, a thread one column.
-constexpr int kDecayTokens = 16;
+// takes 4 tokens (their inner values in LDS) and 256 columns, a thread one column of all 4: its row of w is read
+// in 16-byte pieces where rows allow them.
+constexpr int kDecayTokens = 4;
 template <typename T>
 __global__ void __launch_bounds__(256) decay_lowrank_kernel(float* __restrict__ out, const T* __restrict__ x, long x_stride,
                                                             const T* __restrict__ w, const T* __restrict__ bias, int rows,
-                                                            int N, int R, float inv_tau) {
-  extern __shared__ float xl[];  // [kDecayTokens][R]
+                                                            int N, int R, float inv_tau, int vec) {
+  constexpr int EL = El<T>::N;
+  extern __shared__ float xl[];  // [R][kDecayTokens]
   const int t0 = blockIdx.x * kDecayTokens, nt = min(kDecayTokens, rows - t0);
-  for (int i = threadIdx.x; i < nt * R; i += 256) {
-    const int t = i / R;
-    xl[i] = ldf(x + static_cast<long>(t0 + t) * x_stride + (i - t * R));
+  for (int i = threadIdx.x; i < kDecayTokens * R; i += 256) {
+    const int t = i / R, r = i - t * R;
+    xl[r * kDecayTokens + t] = t < nt ? ldf(x + static_cast<long>(t0 + t) * x_stride + r) : 0.f;
   }
   __syncthreads();
   const int n = blockIdx.y * 256 + threadIdx.x;
   if (n >= N) return;
   const T* wr = w + static_cast<long>(n) * R;
-  float acc[kDecayTokens];
   const float b = ldf(bias + n);
+  float acc[kDecayTokens];
 #pragma unroll
   for (int t = 0; t < kDecayTokens; ++t) acc[t] = b;
-  for (int r = 0; r < R; ++r) {
-    const float wv = ldf(wr + r);
+  if (vec) {
+#pragma unroll 2
+    for (int r = 0; r < R; r += EL) {
+      float wv[EL];
+      load16(wr + r, wv);
 #pragma unroll
-    for (int t = 0; t < kDecayTokens; ++t)
-      if (t < nt) acc[t] += wv * xl[t * R + r];
+      for (int e = 0; e < EL; ++e)
+#pragma unroll
+        for (int t = 0; t < kDecayTokens; ++t) acc[t] += wv[e] * xl[(r + e) * kDecayTokens + t];
+    }
+  } else {
+    for (int r = 0; r < R; ++r) {
+      const float wv = ldf(wr + r);
+#pragma unroll
+      for (int t = 0; t < kDecayTokens; ++t) acc[t] += wv * xl[r * kDecayTokens + t];
+    }
   }
 #pragma unroll
   for (int t = 0; t < kDecayTokens; ++t)
@@ -535,12 +548,13 @@ bool launch_decay_lowrank(float* out, const void* x, long x_stride, const void* 
   const size_t shm = static_cast<size_t>(kDecayTokens) * R * sizeof(float);
   if (shm > 60 * 1024) return false;
   const dim3 grid((rows + kDecayTokens - 1) / kDecayTokens, (N + 255) / 256);
+  const int vec = R % (bf ? 8 : 4) == 0 && reinterpret_cast<uintptr_t>(w) % 16 == 0;
   if (bf)
     hipLaunchKernelGGL(decay_lowrank_kernel<bf16_t>, grid, dim3(256), shm, st, out, (const bf16_t*)x, x_stride, (const bf16_t*)w,
-                       (const bf16_t*)bias, rows, N, R, 1.f / tau);
+                       (const bf16_t*)bias, rows, N, R, 1.f / tau, vec);
   else
     hipLaunchKernelGGL(decay_lowrank_kernel<float>, grid, dim3(256), shm, st, out, (const float*)x, x_stride, (const float*)w,
-                       (const float*)bias, rows, N, R, 1.f / tau);
+                       (const float*)bias, rows, N, R, 1.f / tau, vec);
   MXS_CHECK_LAUNCH();
   return true;
 }

@@ -1,11 +1,12 @@
-"""Prefill and decode throughput of a layer-list design (Voletar, Tapasun, Momuvik, Seradra) beside the models
+"""Prefill and decode throughput of a layer-list design (Voletar, Tapasun, Momuvik, Seradra, Tarorax) beside the models
 closest to it at equal width, depth and feed-forward size (random weights), through the same engine
 path: forced steps of the scheduler, the model runner, paged K/V and state slots, decode through the
 captured graphs.  Voletar stands beside a Llama-shaped model; Tapasun beside Voletar and that model;
 Momuvik beside a Mixtral-shaped model (softmax attention and routed experts of the same sizes); Seradra
-beside Momuvik and that model.
+beside Momuvik and that model; Tarorax beside Tapasun (recurrent layers, short convolutions) and Seradra
+(attention, routed experts).
 
-  python bench.py --mixer-bench [--mixer-design voletar|tapasun|momuvik|seradra] [--mixer-sizes 1024,2048]
+  python bench.py --mixer-bench [--mixer-design voletar|tapasun|momuvik|seradra|tarorax] [--mixer-sizes 1024,2048]
                   [--mixer-prompt 4096] [--mixer-batch 64]
 
 Prints one JSON line per (size, model): prefill tokens/s of one prompt in one step, decode tokens/s
@@ -99,7 +100,28 @@ def seradra_shape(width: int, layers: int = 4, window: int = 1024) -> dict:
             "layers": [kinds[i % 4] for i in range(layers)]}
 
 
+def tarorax_shape(width: int, layers: int = 4) -> dict:
+    """Two residual streams; attention in two maps (64-wide queries and keys per map, 128-wide values, 4 query heads
+    per kv head) on the outside, gated linear attention (64 x 128 heads) between; the first layer's feed-forward is
+    the gated one of 8/3 width, the others eight ungated experts of 2 width, two per token out of the better half."""
+    heads = max(width // 128, 1)
+    att = {"heads": heads, "kv_heads": max(heads // 4, 1), "dim": 64, "vdim": 128, "scale": 0.125, "softcap": 30.0, "diff": 0.5,
+           "conv": 4, "q_temp": {"coef": 0.1, "every": 2048}}
+    gla = {"heads": heads, "dim": 64, "vdim": 128, "tau": 16.0}
+    moe = {"kind": "moe", "expert": {"ff": 2 * width},
+           "router": {"experts": MOE_EXPERTS, "top": MOE_TOP, "groups": {"count": 2, "keep": 1}, "scale": 1.0}}
+    kinds = [{"type": "attention", "mixer": att, "mlp": {"kind": "dense", "ff": (8 * width // 3) // 256 * 256}},
+             {"type": "gla", "mixer": gla, "mlp": moe}, {"type": "gla", "mixer": gla, "mlp": moe},
+             {"type": "attention", "mixer": att, "mlp": moe}]
+    return {"architecture": "Tarorax", "width": width, "vocab": 32000, "norm": {"eps": 1e-5}, "streams": 2,
+            "layers": [kinds[i % 4] for i in range(layers)]}
+
+
 def register(width: int, layers: int, design: str = "voletar") -> tuple:
+    if design == "tarorax":
+        ta = mcfg.tarorax_config(f"tarorax-w{width}", tarorax_shape(width, layers))
+        mcfg.REGISTRY[ta.name.lower()] = ta
+        return (ta.name, register(width, layers, "tapasun")[0], register(width, layers, "seradra")[0])
     if design == "seradra":
         sd = mcfg.seradra_config(f"seradra-w{width}", seradra_shape(width, layers))
         mcfg.REGISTRY[sd.name.lower()] = sd
@@ -496,9 +518,137 @@ def seradra_rooflines(width: int, prompt: int, batch: int, context: int) -> list
     return out
 
 
+def tarorax_rooflines(width: int, prompt: int, batch: int, context: int) -> list:
+    """Tarorax's own kernels alone, at the sizes of tarorax_shape(width): time over roofline time, each beside the
+    like kernel of an existing model: Tapasun's attention with a sink (unwindowed, at the same key bytes and value
+    size), its convolution and its q/k/v preparation for the fused one, its delta-rule scan at the same state size
+    and its gated norm; Momuvik's routed experts and fused residual kernel; the gated SiLU."""
+    from ..models.feedforward import RoutedExperts
+    from ..models.mixers import rotary_frequencies
+    from ..ops import seqmix
+    dev = torch.device("cuda")
+    dt = torch.bfloat16
+    bs, out = 16, []
+    i32 = dict(dtype=torch.int32, device=dev)
+    rnd = lambda *sh: torch.randn(*sh, device=dev).to(dt)  # noqa: E731
+
+    def entry(name, t, flops, peak, bytes_, note):
+        roof = max(flops / peak, bytes_ / PEAK_HBM)
+        out.append({"kernel": name, "width": width, "ms": round(1e3 * t, 4), "roofline_ms": round(1e3 * roof, 4),
+                    "x_roofline": round(t / roof, 1), "counts": note})
+
+    shape = tarorax_shape(width)["layers"]
+    ac, gc, mlp = shape[0]["mixer"], shape[1]["mixer"], shape[1]["mlp"]
+    H, G, dk, dv = ac["heads"], ac["kv_heads"], ac["dim"], ac["vdim"]
+    for mode, T, S, ctx in (("prefill", prompt, 1, prompt), ("decode", batch, batch, context)):
+        n = T // S
+        qsl = torch.arange(0, T + 1, n, **i32)
+        seq = torch.full((S,), ctx, **i32)
+        rows = torch.arange(S, **i32)
+        nb = -(-ctx // bs)
+        bt = torch.arange(S * nb, **i32).view(S, nb)
+        pos = torch.cat([torch.arange(ctx - n, ctx, device=dev) for _ in range(S)])
+        slots = torch.cat([bt[s_].long().repeat_interleave(bs)[ctx - n:ctx] * bs + pos[:n] % bs for s_ in range(S)])
+        keys = ctx if mode == "decode" else ctx / 2
+        # attention in two maps beside one map of twice the query size over the same values
+        kd = 2 * dk
+        cache = rnd(S * nb, G * bs * (kd + dv))
+        voff = G * bs * kd
+        q, gate = rnd(T, H * kd), rnd(T, H * dv)
+        sink = torch.zeros(H, device=dev)
+        kvb = 2.0 * (S * ctx * G * (kd + dv) + 2 * T * H * kd)
+        t = _time(lambda: seqmix.differential_attention(q, cache, bt, qsl, seq, 0, voff, H, G, dk, dv, bs, 0.125, 30.0, 0.4, 0.5, 1e-5,
+                                                        gate, n, ctx, S if n == 1 else 0), 5)
+        entry(f"differential_attention/{mode}", t, 2.0 * T * H * keys * (kd + 2 * dv), PEAK_BF16, kvb + 2.0 * T * H * dv,
+              f"{T} rows x {H} heads x ~{int(keys)} keys of 2 x {dk} + {dv}, both maps' products, bf16 MFMA peak")
+        t = _time(lambda: seqmix.window_attention(q, cache, bt, qsl, seq, 0, voff, H, G, kd, dv, bs, 0.09, 0, 0, max_query_len=n,
+                                                  sink=sink), 5)
+        entry(f"sink_attention/{mode} (tapasun)", t, 2.0 * T * H * keys * (kd + dv), PEAK_BF16, kvb,
+              f"{T} rows x {H} heads x ~{int(keys)} keys of {kd} + {dv}, bf16 MFMA peak")
+        # convolution, query factor and page write in one pass, beside the convolution alone and the page write alone
+        QC, C = H * kd, H * kd + G * (kd + dv)
+        x, wc, bc = rnd(T, C), rnd(4, C), rnd(C)
+        cst = torch.zeros(S, 3 * C, device=dev)
+        t = _time(lambda: seqmix.conv_qkv_cache(x, wc, bc, cst, rows, 0, qsl, seq, pos, slots, cache, 0, voff, QC, G, kd, dv, bs,
+                                                0.1, 2048.0, n), 5)
+        cb = 4.0 * T * C + 24.0 * S * C
+        entry(f"conv_qkv_cache/{mode}", t, 0.0, PEAK_F32, cb, f"{T} rows x {C} channels, 4 taps; rows in, q and pages out")
+        t = _time(lambda: seqmix.causal_conv(x, wc, bc, cst, rows, 0, qsl, seq, silu=False), 5)
+        entry(f"causal_conv/{mode} (tapasun)", t, 0.0, PEAK_F32, cb, f"{T} rows x {C} channels, 4 taps; rows read and written once")
+        fr = rotary_frequencies(64, 500000.0, None).to(dev)
+        k, v = rnd(T, G * kd), rnd(T, G * dv)
+        t = _time(lambda: seqmix.rope_qkv_cache(q, k, v, pos, slots, cache, 0, voff, H, G, kd, dv, bs, fr, None, None, 1e-5, None), 5)
+        entry(f"rope_qkv_cache/{mode} (tapasun)", t, 0.0, PEAK_F32, 4.0 * T * C, f"{T} rows: q read and written, k and v to the pages")
+        # gated linear attention beside the delta rule at the same state size
+        Hg, d1, d2 = gc["heads"], gc["dim"], gc["vdim"]
+        state = torch.zeros(S, Hg * d1 * d2, device=dev)
+        qq, kk, vv, bb = rnd(T, Hg * d1), rnd(T, Hg * d1), rnd(T, Hg * d2), rnd(T, Hg)
+        la = -torch.rand(T, Hg * d1, device=dev) * 0.1
+        sb = 8.0 * S * Hg * d1 * d2 + 2.0 * T * Hg * (2 * d1 + d2) + 4.0 * T * Hg * d2
+        t = _time(lambda: seqmix.gla_scan(qq, kk, vv, la, state, rows, 0, qsl, seq, Hg, d1, d2, d1 ** -0.5, max_query_len=n), 5)
+        entry(f"gla_scan/{mode}", t, 5.0 * T * Hg * d1 * d2, PEAK_F32, sb + 4.0 * T * Hg * d1,
+              f"{T} rows x {Hg} heads x {d1}x{d2} state, fp32 peak; state read and written once")
+        aa, hb, cbias = rnd(T, Hg * d1), torch.zeros(Hg, device=dev), torch.zeros(Hg * d1, device=dev)
+        t = _time(lambda: seqmix.delta_scan(qq, kk, vv, bb, aa, cbias, hb, state, rows, 0, qsl, seq, Hg, Hg, d1, d2, d1 ** -0.5,
+                                            max_query_len=n), 5)
+        entry(f"delta_scan/{mode} (tapasun)", t, 7.0 * T * Hg * d1 * d2, PEAK_F32, sb + 2.0 * T * Hg * d1,
+              f"{T} rows x {Hg} heads x {d1}x{d2} state, fp32 peak; state read and written once")
+        x1, w2, b2 = rnd(T, 16), rnd(Hg * d1, 16), rnd(Hg * d1)
+        t = _time(lambda: seqmix.decay_lowrank(x1, w2, b2, 16.0), 5)
+        entry(f"decay_lowrank/{mode}", t, 32.0 * T * Hg * d1, PEAK_F32, 4.0 * T * Hg * d1 + 32.0 * (T + Hg * d1),
+              f"{T} rows x {Hg * d1} channels from 16 inner values, fp32 out")
+        hx, wr = rnd(T, width), rnd(MOE_EXPERTS, width)
+        t = _time(lambda: seqmix.gate_linear(hx, wr, None), 5)
+        entry(f"gate_linear/{mode} (momuvik)", t, 2.0 * T * width * MOE_EXPERTS, PEAK_F32, 2.0 * T * width,
+              f"{T} rows x {width} to {MOE_EXPERTS} fp32 columns")
+        o, gg, wn = torch.randn(T, Hg * d2, device=dev), rnd(T, Hg * d2), rnd(d2)
+        t = _time(lambda: seqmix.gated_norm(o, gg, wn, 1e-5, Hg, "silu", False, dt), 5)
+        entry(f"gated_norm/{mode}", t, 0.0, PEAK_F32, 8.0 * T * Hg * d2, f"{T} rows x {Hg * d2}: fp32 in, gate in, bf16 out")
+        # routed experts: ungated units of 2 width (two products) beside capped gated ones of 4/3 width (three)
+        E, top, ff = MOE_EXPERTS, MOE_TOP, mlp["expert"]["ff"]
+        ff3 = (4 * width // 3) // 256 * 256
+        act = min(E, T * top)
+        r = mlp["router"]
+        fu = RoutedExperts("f.", width, E, top, ff, None, renorm=True, weigh="output", gated=False, act="gelu_erf", correction=True,
+                           groups=r["groups"]["count"], keep=r["groups"]["keep"], scale=r["scale"])
+        w = {"f.router": wr, "f.correction": torch.zeros(E, device=dev), "f._in": rnd(E, width, ff) * width ** -0.5,
+             "f._down": rnd(E, ff, width) * ff ** -0.5}
+        t = _time(lambda: fu.forward(hx, w), 5)
+        entry(f"routed_experts/{mode}", t, 4.0 * T * top * width * ff, PEAK_BF16, 2.0 * (2 * act * width * ff + 2 * T * width),
+              f"{T} rows x {top} of {E} ungated experts of {ff}, bf16 MFMA peak; {act} experts' weights read once")
+        fm = RoutedExperts("f.", width, E, top, ff3, 7.0)
+        w = {"f.router": wr, "f._in": rnd(E, width, 2 * ff3) * width ** -0.5, "f._down": rnd(E, ff3, width) * ff3 ** -0.5}
+        t = _time(lambda: fm.forward(hx, w), 5)
+        entry(f"routed_experts/{mode} (momuvik)", t, 6.0 * T * top * width * ff3, PEAK_BF16,
+              2.0 * (3 * act * width * ff3 + 2 * T * width), f"{T} rows x {top} of {E} gated experts of {ff3}, bf16 MFMA peak")
+        lg, corr = torch.randn(T, E, device=dev), torch.zeros(E, device=dev)
+        t = _time(lambda: seqmix.route_topk(lg, top, True, correction=corr, groups=2, keep=1, scale=1.5), 5)
+        entry(f"route_grouped/{mode}", t, 0.0, PEAK_F32, 4.0 * T * (E + 2 * top), f"{T} rows x {E} logits")
+        t = _time(lambda: seqmix.route_topk(lg, top), 5)
+        entry(f"route_topk/{mode} (momuvik)", t, 0.0, PEAK_F32, 4.0 * T * (E + 2 * top), f"{T} rows x {E} logits")
+        # activations, streams
+        z = rnd(T, 4 * width)
+        t = _time(lambda: seqmix.unary_act(z, "gelu_erf"), 5)
+        entry(f"gelu/{mode}", t, 0.0, PEAK_F32, 4.0 * T * 4 * width, f"{T} rows x {4 * width}: in and out")
+        t = _time(lambda: seqmix.act_mul(z, "gelu_tanh"), 5)
+        entry(f"gelu_mul/{mode}", t, 0.0, PEAK_F32, 3.0 * T * 4 * width, f"{T} rows x {2 * width}: gate and up in, product out")
+        t = _time(lambda: seqmix.silu_mul(z), 5)
+        entry(f"silu_mul/{mode} (tapasun)", t, 0.0, PEAK_F32, 3.0 * T * 4 * width, f"{T} rows x {2 * width}: gate and up in, product out")
+        X, a, ow = torch.randn(T, 2, width, device=dev), rnd(T, width), torch.zeros(width, device=dev).to(dt)
+        cf = torch.tensor([1.0, 0.0, 0.0, 1.0, 0.1, 0.1, 0.5, 0.5], device=dev)
+        t = _time(lambda: seqmix.streams_update(X, a, cf, 1e-5, ow, dt, scale=ow, w_offset=1.0), 5)
+        entry(f"streams_update/{mode}", t, 0.0, PEAK_F32, T * width * (2 * 8.0 + 2.0 + 2.0),
+              f"{T} rows x {width}: two fp32 streams in and out, branch in, normed bf16 out")
+        x = torch.randn(T, width, device=dev)
+        t = _time(lambda: seqmix.resid_update(x, a, 1e-5, norm_w=ow, out_dtype=dt, w_offset=1.0), 5)
+        entry(f"resid_update/{mode} (momuvik)", t, 0.0, PEAK_F32, T * width * (4.0 + 2.0 + 4.0 + 2.0),
+              f"{T} rows x {width}: stream in and out, branch in, normed bf16 out")
+    return out
+
+
 def main(sizes: list, prompt: int, batch: int, context: int, layers: int = 4, only: str = "all",
          design: str = "voletar") -> int:
-    """only: all | seradra | momuvik | mixtral | tapasun | voletar | llama | kernels (e.g. one model alone under a profiler)."""
+    """only: all | tarorax | seradra | momuvik | mixtral | tapasun | voletar | llama | kernels (e.g. one model alone under a profiler)."""
     from .. import ops
     ops.ext()
     for width in sizes:
@@ -507,7 +657,9 @@ def main(sizes: list, prompt: int, batch: int, context: int, layers: int = 4, on
             if only in ("all", name.split("-")[0]):
                 print(json.dumps(run_model(name, prompt, batch, context)), flush=True)
         if only in ("all", "kernels"):
-            if design == "seradra":
+            if design == "tarorax":
+                rows = tarorax_rooflines(width, prompt, batch, context)
+            elif design == "seradra":
                 rows = seradra_rooflines(width, prompt, batch, context)
             elif design == "momuvik":
                 rows = momuvik_rooflines(width, prompt, batch, context)

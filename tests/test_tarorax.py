@@ -1,0 +1,781 @@
+"""Tarorax through the engine (residual streams, paged keys / values, state slots, forced and scheduled
+steps) against the plain float64 oracle of tests/tarorax_oracle.py: on the PyTorch forms of the ops here,
+on the HIP kernels under `-m gpu`.  Every test makes its own small configuration and random weights."""
+import math
+import types
+
+import numpy as np
+import pytest
+import torch
+
+from tests import tarorax_oracle as ao
+from tests.tarorax_utils import (BASE, config, cut, dense, diff_attention, engine, gla, layer, moe, rel_err, replay,
+                                 write_checkpoint)
+
+DEVS = ["cpu", pytest.param("cuda", marks=pytest.mark.gpu)]
+DEV_DTYPE = [("cpu", torch.float32), pytest.param("cuda", torch.float32, marks=pytest.mark.gpu),
+             pytest.param("cuda", torch.bfloat16, marks=pytest.mark.gpu)]
+DEV_DTYPE_TOL = [("cpu", "float32", 1e-4), pytest.param("cuda", "float32", 1e-4, marks=pytest.mark.gpu),
+                 pytest.param("cuda", "bfloat16", 0.1, marks=pytest.mark.gpu)]
+EPS = 1e-5
+CLOSE = 0.02  # a routing margin below this may fall either way in bf16
+
+
+def _skip(dev):
+    if dev == "cuda" and not torch.cuda.is_available():
+        pytest.skip("no GPU")
+
+
+def _tokens(n, vocab, seed):
+    return np.random.default_rng(seed).integers(0, vocab, n).tolist()
+
+
+def _row_errors(got, want):
+    d = got - want
+    d = d - d.mean(-1, keepdims=True)
+    return np.sqrt((d ** 2).mean(-1)) / np.sqrt((want ** 2).mean())
+
+
+def _check(got, want, tol, margins=None):
+    """fp32 (tol well below 1e-2): every row within tol.  bf16: the mean over the rows (of eight or more)
+    within tol / 4 and the worst row within 2.5 tol -- up to the sequence's first token whose routing was a
+    close call in the oracle: rounding may send that token to another expert, and later tokens read what it
+    left in pages and states.  From there on the rows must stay near (median within tol, none beyond 1)."""
+    if tol < 1e-2:
+        e = rel_err(got, want)
+        assert e < tol, f"relative error {e:.3g} >= {tol}"
+        return
+    e = _row_errors(got, want)
+    assert np.isfinite(e).all()
+    if margins is not None and (np.asarray(margins) < CLOSE).any():
+        first = int(np.argmax(np.asarray(margins) < CLOSE))
+        after = e[first:]
+        assert np.median(after) < tol and after.max() < 1.0, f"rows after a close call: median {np.median(after):.3g}, worst {after.max():.3g}"
+        e = e[:first]
+    assert (len(e) < 8 or e.mean() < tol / 4) and (len(e) == 0 or e.max() < 2.5 * tol), \
+        f"row errors: mean {e.mean():.3g}, worst {e.max():.3g} (tol {tol})"
+
+
+def _oracle_model(cfg, w, tokens):
+    m = []
+    lg, _ = ao.run(cfg, w, tokens, m)
+    return lg, m
+
+
+# ----------------------------------------------------------------------------- the mixers alone
+def _mixer_setup(kind, mc, width, seed=0):
+    from mxserve.models.tarorax import build_mixer
+    m = build_mixer(kind, "m.", width, mc)
+    g = torch.Generator().manual_seed(seed)
+    shapes = {name: (rows, width) for name, rows in m.proj_rows()}
+    shapes.update(m.extra_shapes())
+    w = {k: torch.randn(s, generator=g) * (s[-1] ** -0.5 if len(s) > 1 else 1.0) for k, s in shapes.items()}
+    for k in w:
+        if k.endswith(".norm"):
+            w[k] = 1.0 + 0.2 * w[k]
+        elif k.endswith("a2.b"):
+            w[k] = 1.0 + 2.0 * w[k]
+        elif k.endswith(".b"):
+            w[k] = 0.5 * w[k]
+        elif k.endswith(("lq1", "lk1", "lq2", "lk2")):
+            w[k] = w[k] * w[k].numel() ** -0.5
+    return m, w
+
+
+class _Pages:
+    """One sequence's pages and state slot, scattered over pools that hold stale numbers (also NaN)."""
+
+    def __init__(self, T, elems, state_floats, dev, dtype, bs=16, slot=2):
+        nb = -(-T // bs) + 3
+        self.bs, self.dev, self.slot = bs, dev, slot
+        self.cache = torch.randn(nb, elems + 16, device=dev).to(dtype)
+        self.cache[:, ::7] = float("nan")
+        self.state = torch.full((4, state_floats + 9), float("nan"), device=dev)
+        self.blocks = torch.randperm(nb, generator=torch.Generator().manual_seed(3))[:-(-T // bs)].to(torch.int32)
+
+    def ctx(self, at, n):
+        from mxserve.models.mixers import StepContext
+        dev, bs = self.dev, self.bs
+        pos = torch.arange(at, at + n)
+        md = types.SimpleNamespace(
+            positions=pos.to(dev), slot_mapping=(self.blocks[pos // bs].long() * bs + pos % bs).to(dev),
+            block_tables=self.blocks[None].to(dev), query_start_loc=torch.tensor([0, n], dtype=torch.int32, device=dev),
+            seq_lens=torch.tensor([at + n], dtype=torch.int32, device=dev), max_query_len=n, max_seq_len=at + n,
+            num_decodes=1 if n == 1 else 0, state_rows=torch.tensor([self.slot], dtype=torch.int32, device=dev))
+        return StepContext(md=md, cache=self.cache, state=self.state, block_size=bs, eps=EPS)
+
+
+def _run_mixer(m, w, h, dev, portions, dtype=torch.float32, koff=8, soff=4):
+    """The mixer over one sequence cut into portions; pages and state start at an offset."""
+    T = h.shape[0]
+    wt = {k: v.to(dev).to(dtype) for k, v in w.items()}
+    w_in = torch.cat([wt[name] for name, _ in m.proj_rows()])
+    if hasattr(m, "finish_weights"):
+        m.finish_weights(wt)
+    elems = 16 * m.kv_heads * (m.dk + m.dv)
+    voff = koff + 16 * m.kv_heads * m.dk
+    pg = _Pages(T, koff + elems, soff + m.state_floats, dev, dtype)
+    outs, at, i = [], 0, 0
+    while at < T:
+        n = min(portions[min(i, len(portions) - 1)], T - at)
+        i += 1
+        hp = h[at:at + n].to(dev).to(dtype)
+        y = hp @ w_in.T
+        parts, c = [], 0
+        for _, rows in m.proj_rows():
+            parts.append(y[:, c:c + rows])
+            c += rows
+        o = m.forward(parts, hp, wt, pg.ctx(at, n), koff, voff, soff)
+        outs.append(o + wt[m.out_bias] if m.out_bias else o)
+        at += n
+    return torch.cat(outs).double().cpu().numpy()
+
+
+def _oracle_mixer(kind, mc, w, h):
+    wn = {k: v.double().numpy() for k, v in w.items()}
+    cls = {"attention": ao.DifferentialAttention, "gla": ao.GatedLinearAttention}[kind]
+    o = cls(mc, wn, "m.", EPS)
+    hn = h.double().numpy()
+    return np.stack([o.step(hn[t], t) for t in range(h.shape[0])])
+
+
+def _bf(w, h):
+    """Weights and inputs rounded to bf16, so that the oracle and a bf16 run start from the same numbers."""
+    return {k: v.to(torch.bfloat16).float() for k, v in w.items()}, h.to(torch.bfloat16).float()
+
+
+def _check_bf16(got, want, what):
+    """Most rows near, none by much on average: a head whose sum all but cancels (its unit norm blows rounding up, or
+    turns its sign) may take one row far off."""
+    e = _row_errors(got, want)
+    assert np.isfinite(e).all() and np.quantile(e, 0.95) < 0.08 and e.mean() < 0.03, (what, e.max(), e.mean())
+
+
+def _compare(kind, shapes, width, h, dev, dtype, portions):
+    for n, mc in enumerate(shapes):
+        m, w = _mixer_setup(kind, mc, width, seed=n)
+        if dtype == torch.bfloat16:
+            w, hh = _bf(w, h)
+            _check_bf16(_run_mixer(m, w, hh, dev, portions, dtype), _oracle_mixer(kind, mc, w, hh), mc)
+        else:
+            _check(_run_mixer(m, w, h, dev, portions), _oracle_mixer(kind, mc, w, h), 1e-4)
+
+
+PORTIONS = [[1000], [1], [2], [5, 1, 9, 2, 30]]
+ATTENTION_SHAPES = [
+    diff_attention(),
+    diff_attention(heads=1, kv_heads=1, dim=1, vdim=3, scale=0.7, softcap=3.0, diff=0.0, conv=1, coef=0.0, every=1),
+    diff_attention(heads=4, kv_heads=2, dim=8, vdim=12, scale=0.4, softcap=500.0, diff=0.8, conv=2, every=1),
+    diff_attention(heads=5, kv_heads=5, dim=32, vdim=64, scale=0.2, softcap=40.0, conv=6, every=50),
+    diff_attention(heads=3, kv_heads=1, dim=10, vdim=7, scale=0.3, conv=4),
+    diff_attention(heads=40, kv_heads=1, dim=16, vdim=16, scale=0.25, conv=2),
+    diff_attention(heads=4, kv_heads=2, dim=64, vdim=128, scale=0.1, softcap=8.0),
+    diff_attention(heads=2, kv_heads=1, dim=104, vdim=200, scale=0.1, conv=3),
+    diff_attention(heads=2, kv_heads=2, dim=136, vdim=264, scale=0.08, softcap=70.0, conv=2),
+]
+
+
+@pytest.mark.parametrize("dev,dtype", DEV_DTYPE)
+@pytest.mark.parametrize("portions", PORTIONS)
+def test_differential_attention_mixer(dev, dtype, portions):
+    """Grouped heads; one head of one dimension without filter; bounds that need a running maximum; one kv
+    head per head; sizes that fit no vector load; more query heads per kv head than a tile has columns; wide
+    heads; heads wider than the matrix-core form takes; filters longer than most portions."""
+    _skip(dev)
+    h = torch.randn(70, 72, generator=torch.Generator().manual_seed(1))
+    _compare("attention", ATTENTION_SHAPES, 72, h, dev, dtype, portions)
+
+
+@pytest.mark.parametrize("dev,dtype", DEV_DTYPE)
+@pytest.mark.parametrize("portions", [[1000], [130, 1, 1, 200], [33, 2, 64, 127, 1, 129]])
+def test_differential_attention_over_many_tiles(dev, dtype, portions):
+    """Contexts of several key tiles, which few-row steps also split over workgroups."""
+    _skip(dev)
+    h = torch.randn(390, 40, generator=torch.Generator().manual_seed(2))
+    _compare("attention", [diff_attention(heads=4, kv_heads=1, dim=16, vdim=36, conv=4),
+                           diff_attention(heads=2, kv_heads=2, dim=40, vdim=72, softcap=90.0, conv=2)], 40, h, dev, dtype, portions)
+
+
+GLA_SHAPES = [gla(), gla(heads=1, dim=1, vdim=2, tau=1.0), gla(heads=4, dim=16, vdim=40, tau=16.0), gla(heads=2, dim=33, vdim=7, tau=0.5),
+              gla(heads=5, dim=64, vdim=64, tau=30.0), gla(heads=2, dim=96, vdim=80, tau=8.0), gla(heads=1, dim=200, vdim=20, tau=5.0)]
+
+
+@pytest.mark.parametrize("dev,dtype", DEV_DTYPE)
+@pytest.mark.parametrize("portions", PORTIONS)
+def test_gated_linear_attention_mixer(dev, dtype, portions):
+    """Key and value sizes apart, one head of one channel, roots below and above one, key sizes that are no
+    multiple of the lane runs."""
+    _skip(dev)
+    h = torch.randn(70, 72, generator=torch.Generator().manual_seed(1))
+    _compare("gla", GLA_SHAPES, 72, h, dev, dtype, portions)
+
+
+@pytest.mark.parametrize("dev,dtype", DEV_DTYPE)
+@pytest.mark.parametrize("portions", [[1000], [17, 300, 1, 1, 200], [129, 128, 127]])
+def test_gated_linear_attention_long_chunks(dev, dtype, portions):
+    """Chunks that the GPU scan cuts into pieces, with decays slow enough that what a piece inherits matters to
+    its end, fast ones that forget within a token, and both in one head."""
+    _skip(dev)
+    h = torch.randn(530, 48, generator=torch.Generator().manual_seed(4))
+    for n, (mc, lo, hi) in enumerate([(gla(heads=2, dim=16, vdim=24, tau=16.0), 2.0, 6.0), (gla(heads=1, dim=40, vdim=18, tau=1.0), -40.0, 8.0),
+                                      (gla(heads=3, dim=64, vdim=32, tau=4.0), -100.0, -10.0)]):
+        m, w = _mixer_setup("gla", mc, 48, seed=n)
+        w["m.a2.b"] = lo + (hi - lo) * torch.rand(w["m.a2.b"].shape, generator=torch.Generator().manual_seed(9))
+        if dtype == torch.bfloat16:
+            w, hh = _bf(w, h)
+            _check_bf16(_run_mixer(m, w, hh, dev, portions, dtype), _oracle_mixer("gla", mc, w, hh), mc)
+        else:
+            _check(_run_mixer(m, w, h, dev, portions), _oracle_mixer("gla", mc, w, h), 1e-4)
+
+
+def test_low_rank_size_comes_from_the_tensors(tmp_path):
+    """The inner size of the decay's low-rank pair is in no config entry."""
+    cfg = config([layer(gla(heads=2, dim=8, vdim=8), None)], width=24, vocab=30, streams=2)
+
+    def tweak(sd):
+        g = torch.Generator().manual_seed(1)
+        sd["l0.mix.a1"] = torch.randn(5, 24, generator=g).to(torch.bfloat16)
+        sd["l0.mix.a2"] = torch.randn(16, 5, generator=g).to(torch.bfloat16)
+
+    w = write_checkpoint(tmp_path, cfg, seed=3, tweak=tweak)
+    t = _tokens(20, 30, 4)
+    eng = engine(tmp_path, "cpu", "float32", max_tokens=64)
+    _check(replay(eng, [[("a", t, True)]])["a"], ao.run(cfg, w, t)[0], 1e-4)
+
+
+# ----------------------------------------------------------------------------- single mechanisms
+def _picking(scale=1.0, cap=30.0, conv=1, heads=1, diff=0.5, shift=0):
+    """Every head's first map: the query reads h[:8], the key h[8:16]; its second map asks for nothing (equal weights);
+    the value is h[16:24].  The filter passes the value of `shift` tokens ago."""
+    mc = diff_attention(heads=heads, kv_heads=1, dim=8, vdim=8, scale=scale, softcap=cap, diff=diff, conv=conv, coef=0.0, every=1)
+    from mxserve.models.tarorax import build_mixer
+    m = build_mixer("attention", "m.", 24, mc)
+    eye, z = torch.eye(8), torch.zeros(8, 8)
+    tap = torch.zeros(1, conv)
+    tap[0, conv - 1 - shift] = 1.0
+    own = torch.zeros(1, conv)
+    own[0, conv - 1] = 1.0
+    w = {"m.q": torch.cat([torch.cat([eye, z, z], 1), torch.zeros(8, 24)] * heads), "m.k": torch.cat([torch.cat([z, eye, z], 1), torch.zeros(8, 24)]),
+         "m.v": torch.cat([z, z, eye], 1), "m.g": torch.zeros(8 * heads, 24), "m.q.b": torch.zeros(16 * heads), "m.k.b": torch.zeros(16),
+         "m.v.b": torch.zeros(8), "m.q.conv": own.repeat(16 * heads, 1), "m.k.conv": tap.repeat(16, 1), "m.v.conv": tap.repeat(8, 1),
+         "m.lq1": torch.zeros(8), "m.lk1": torch.zeros(8), "m.lq2": torch.zeros(8), "m.lk2": torch.zeros(8),
+         "m.o": torch.cat([torch.eye(8 * heads)[:, :], torch.zeros(max(0, 24 - 8 * heads), 8 * heads)])[:24], "m.o.b": torch.zeros(24)}
+    return mc, m, w
+
+
+@pytest.mark.parametrize("dev,dtype", DEV_DTYPE)
+@pytest.mark.parametrize("back", [0, 1, 12, 13, 14, 28, 29, 60, 61, 127, 128, 172, 173, 236, 237, 299, 300])
+def test_one_far_key_stands_out(dev, dtype, back):
+    """One key among three hundred matches the last query: the query's own position, both sides of page and tile
+    borders, and the sequence's first tokens, in a whole prompt, when the last token is decoded alone, and in
+    uneven portions.  The output is that key's value less lambda times the mean of all."""
+    _skip(dev)
+    T = 301
+    mc, m, w = _picking(scale=1.0, cap=30.0)
+    target = T - 1 - back
+    g = torch.Generator().manual_seed(5)
+    h = 0.1 * torch.randn(T, 24, generator=g)
+    h[target, 13] += 6.0
+    h[T - 1, :8] = 0.0
+    h[T - 1, 5] = 6.0
+    h[:, 16:] = torch.randn(T, 8, generator=g)
+    h[target, 16:] = torch.tensor([3.0, -3.0, 3.0, 3.0, -3.0, -3.0, 3.0, -3.0])
+    h = h.to(torch.bfloat16).float()
+    want = _oracle_mixer("attention", mc, w, h)
+    o = h[target, 16:].double().numpy() - 0.5 * h[:, 16:].double().numpy().mean(0)
+    assert np.abs(want[T - 1, :8] - 0.25 * o / np.sqrt((o ** 2).mean())).max() < 0.01  # the oracle itself shows the case
+    for portions in ([T], [T - 1, 1], [7, 2, 160, 3, 100, 1]):
+        got = _run_mixer(m, dict(w), h, dev, portions, dtype)
+        assert np.abs(got - want).max() < (1e-4 if dtype == torch.float32 else 0.01)
+
+
+@pytest.mark.parametrize("dev", DEVS)
+def test_first_tokens_see_no_filtered_bias(dev):
+    """Before a sequence's start the filter's inputs are zero, not the bias: with zero projections the output at
+    token t is the bias times the sum of the taps that reach a token, in any cut."""
+    _skip(dev)
+    mc, m, w = _picking(conv=4)
+    for k in ("m.q", "m.k", "m.v"):
+        w[k] = torch.zeros_like(w[k])
+    b = torch.tensor([1.0, -2.0, 0.5, 3.0, -1.0, 0.25, 2.0, -0.5])
+    taps = torch.tensor([0.5, -1.0, 0.25, 2.0])
+    w["m.v.b"] = b
+    w["m.v.conv"] = taps.repeat(8, 1)
+    T = 12
+    h = torch.randn(T, 24, generator=torch.Generator().manual_seed(3))
+    v = [float(taps[max(0, 3 - t):].sum()) for t in range(T)]  # value = v[t] b
+    run = np.cumsum(v) / np.arange(1, T + 1)                   # equal weights; both maps alike: (1 - lambda) times the mean
+    unit = b.double().numpy() / np.sqrt((b.double().numpy() ** 2).mean())
+    want = np.stack([np.sign(r * 0.5) * unit * 0.5 * 0.5 for r in run])
+    for portions in ([T], [1], [2], [3, 1, 5]):
+        assert np.abs(_run_mixer(m, dict(w), h, dev, portions)[:, :8] - want).max() < 1e-4
+
+
+@pytest.mark.parametrize("dev", DEVS)
+def test_filter_reaches_exactly_its_taps_back(dev):
+    """A filter that passes only its oldest tap: keys and values are those of taps - 1 tokens ago, across portions
+    shorter than the filter, single tokens, and a page border."""
+    _skip(dev)
+    for conv in (2, 3, 5):
+        mc, m, w = _picking(conv=conv, shift=conv - 1)
+        h = torch.randn(40, 24, generator=torch.Generator().manual_seed(conv))
+        want = _oracle_mixer("attention", mc, w, h)
+        for portions in ([40], [1], [2], [15, 1, 1, 2, 30]):
+            _check(_run_mixer(m, dict(w), h, dev, portions), want, 1e-4)
+
+
+@pytest.mark.parametrize("dev", DEVS)
+def test_query_factor_steps_with_the_position(dev):
+    """Query columns (keys and values not) times 1 + coef ln(floor((p + 1) / every) + 1): one below `every`, a step
+    at every - 1 and at each multiple, also far out."""
+    _skip(dev)
+    from mxserve.ops import seqmix
+    coef, every = 0.3, 5.0
+    pos = torch.tensor([0, 3, 4, 8, 9, 13, 14, 4998, 4999, 100003])
+    T, QC, G, dk, dv = len(pos), 6, 1, 4, 3
+    C = QC + G * (dk + dv)
+    x = torch.ones(T, C)
+    cache = torch.zeros(8, 16 * (dk + dv))
+    slots = torch.arange(T)
+    md = [t.to(dev) for t in (torch.arange(T, dtype=torch.int32), torch.arange(T + 1, dtype=torch.int32), torch.full((T,), 7, dtype=torch.int32),
+                              pos, slots)]
+    cd = cache.to(dev)
+    q = seqmix.conv_qkv_cache(x.to(dev), torch.ones(1, C).to(dev), None, torch.zeros(T, 4).to(dev), md[0], 0, md[1], md[2], md[3], md[4], cd,
+                              0, 16 * dk, QC, G, dk, dv, 16, coef, every, 1)
+    want = np.array([ao.query_temperature(int(p), coef, every) for p in pos])
+    assert want[0] == want[1] == 1.0 and want[2] > 1.2 and want[2] == want[3] and want[4] > want[3]
+    assert np.abs(q.double().cpu().numpy() - want[:, None]).max() < 1e-5
+    assert torch.equal(cd[0, :T * dk].cpu(), torch.ones(T * dk)) and torch.equal(cd[0, 16 * dk:16 * dk + T * dv].cpu(), torch.ones(T * dv))
+
+
+@pytest.mark.parametrize("dev,dtype", DEV_DTYPE)
+@pytest.mark.parametrize("cap", [0.5, 6.0, 30.0, 59.0, 61.0, 300.0])
+def test_scores_are_bounded(dev, dtype, cap):
+    """Scores far beyond the bound in both directions: the weights of the strongest and the weakest key differ by
+    e^(2 cap) at most; small bounds keep every key in play."""
+    _skip(dev)
+    mc, m, w = _picking(scale=2.0, cap=cap)
+    h = torch.randn(90, 24, generator=torch.Generator().manual_seed(8))
+    h[:, :16] *= 3.0
+    h = h.to(torch.bfloat16).float()
+    want = _oracle_mixer("attention", mc, w, h)
+    for portions in ([90], [50, 1, 3, 1, 35]):
+        got = _run_mixer(m, dict(w), h, dev, portions, dtype)
+        assert np.abs(got - want).max() < (2e-4 if dtype == torch.float32 else 0.02)
+
+
+def test_bound_and_difference_show_in_the_oracle():
+    """Without the bound, or without the second map, the crafted case above comes out otherwise."""
+    mc, _, w = _picking(scale=2.0, cap=6.0)
+    h = torch.randn(90, 24, generator=torch.Generator().manual_seed(8))
+    h[:, :16] *= 3.0
+    want = _oracle_mixer("attention", mc, w, h)
+    assert np.abs(_oracle_mixer("attention", dict(mc, softcap=1e6), w, h) - want).max() > 0.05
+    assert np.abs(_oracle_mixer("attention", dict(mc, diff=0.0), w, h) - want).max() > 0.05
+
+
+def test_lambda_is_one_number_of_the_layer():
+    mc = diff_attention(diff=0.3)
+    m, w = _mixer_setup("attention", mc, 40)
+    want = math.exp(float(w["m.lq1"].double() @ w["m.lk1"].double())) - math.exp(float(w["m.lq2"].double() @ w["m.lk2"].double())) + 0.3
+    m.finish_weights({k: v.clone() for k, v in w.items()})
+    assert abs(m.lam - want) < 1e-6
+
+
+@pytest.mark.parametrize("dev", DEVS)
+def test_decay_forgets_channel_by_channel(dev):
+    """Two key channels, one that never decays and one that is gone after a token: what was written through the
+    first is read hundreds of tokens later, what was written through the second is not."""
+    _skip(dev)
+    from mxserve.ops import seqmix
+    T, H, dk, dv = 300, 1, 2, 3
+    q, k, v = torch.ones(T, 2), torch.zeros(T, 2), torch.zeros(T, 3)
+    k[3], v[3] = torch.tensor([1.0, 1.0]), torch.tensor([1.0, 2.0, 3.0])
+    la = torch.tensor([0.0, -60.0]).repeat(T, 1)
+    state = torch.full((2, 8), float("nan"))
+    i32 = lambda *x: torch.tensor(x, dtype=torch.int32).to(dev)  # noqa: E731
+    st = state.to(dev)
+    o = seqmix.gla_scan(q.to(dev), k.to(dev), v.to(dev), la.to(dev), st, i32(1), 1, i32(0, T), i32(T), H, dk, dv, 0.5, max_query_len=T).cpu()
+    assert torch.equal(o[:3], torch.zeros(3, 3)) and torch.allclose(o[3], torch.tensor([1.0, 2.0, 3.0]))
+    assert torch.allclose(o[4:], torch.tensor([0.5, 1.0, 1.5]).expand(T - 4, 3))
+    assert torch.allclose(st[1, 1:7].cpu().view(3, 2)[:, 0], torch.tensor([1.0, 2.0, 3.0])) and bool(torch.isnan(st[0]).all())
+
+
+# ----------------------------------------------------------------------------- feed-forwards
+def _ff_setup(mlp, width, seed=0, router_gain=3.0):
+    from mxserve.models.tarorax import build_ff
+    f = build_ff("f.", width, mlp)
+    g = torch.Generator().manual_seed(seed)
+    w = {k: torch.randn(s, generator=g) * (s[-1] ** -0.5 if len(s) > 1 else 0.3) for k, s in f.shapes().items()}
+    if "f.router" in w:
+        w["f.router"] = w["f.router"] * router_gain
+    return f, w
+
+
+@pytest.mark.parametrize("dev", DEVS)
+def test_both_forms_of_gelu(dev):
+    """Near zero, at zero, where the two forms differ most, and far out; with and without a gate; widths of whole
+    16-byte pieces and others."""
+    _skip(dev)
+    from mxserve.ops import seqmix
+    z = torch.cat([torch.linspace(-12, 12, 241), torch.tensor([0.0, -0.0, 1e-6, -1e-6, 2.0, -2.0, 60.0])])
+    zn = z.double().numpy()
+    assert np.abs(ao.gelu_erf(zn) - ao.gelu_tanh(zn)).max() > 3e-4
+    for kind, ref in (("gelu_erf", ao.gelu_erf), ("gelu_tanh", ao.gelu_tanh), ("silu", ao.silu)):
+        for n in (248, 62, 1):
+            x = z.view(-1, n).to(dev)
+            assert np.abs(seqmix.unary_act(x, kind).double().cpu().numpy() - ref(zn).reshape(-1, n)).max() < 1e-5
+        gu = torch.stack([z, torch.flip(z, [0])], 1).reshape(4, -1)
+        got = seqmix.act_mul(gu.to(dev), kind).double().cpu().numpy()
+        gn = gu.double().numpy()
+        half = gn.shape[1] // 2
+        want = ref(gn[:, :half]) * gn[:, half:]
+        assert np.abs(got - want).max() < 1e-5 * np.abs(want).max()
+    f, w = _ff_setup(dense(40), 24, seed=3)
+    h = 2.0 * torch.randn(9, 24, generator=torch.Generator().manual_seed(1))
+    wn = {k: v.double().numpy() for k, v in w.items()}
+    want = np.stack([ao.dense_ff(x, wn, "f.") for x in h.double().numpy()])
+    wt = {k: v.to(dev) for k, v in w.items()}
+    f.finish_weights(wt)
+    assert np.abs(f.forward(h.to(dev), wt).double().cpu().numpy() - want).max() < 1e-4 * max(1.0, np.abs(want).max())
+
+
+@pytest.mark.parametrize("dev", DEVS)
+@pytest.mark.parametrize("T", [1, 5, 33, 150])
+def test_routed_experts_alone(dev, T):
+    """Both ways through the experts (batched over all experts for a few tokens, sorted rows otherwise); one
+    group, groups of one expert, all groups kept, all experts of the kept group chosen, many experts."""
+    _skip(dev)
+    width = 48
+    h = 1.5 * torch.randn(T, width, generator=torch.Generator().manual_seed(T))
+    for mlp in (moe(), moe(experts=5, top=1, ff=24, groups=1, keep=1), moe(experts=6, top=2, ff=16, groups=6, keep=2, scale=1.0),
+                moe(experts=8, top=4, ff=72, groups=2, keep=1, scale=3.0), moe(experts=70, top=4, ff=16, groups=7, keep=7),
+                moe(experts=140, top=6, ff=8, groups=70, keep=5)):
+        f, w = _ff_setup(mlp, width)
+        wn = {k: v.double().numpy() for k, v in w.items()}
+        want = np.stack([ao.routed_ff(x, wn, "f.", mlp)[0] for x in h.double().numpy()])
+        wt = {k: v.to(dev) for k, v in w.items()}
+        f.finish_weights(wt)
+        got = f.forward(h.to(dev), wt).double().cpu().numpy()
+        assert np.abs(got - want).max() < 2e-4 * max(1.0, np.abs(want).max())
+
+
+def _logit(s):
+    return math.log(s / (1.0 - s))
+
+
+@pytest.mark.parametrize("dev", DEVS)
+def test_group_limited_choice_by_hand(dev):
+    """The correction decides the choice and not the weights; a group counts by its two best; the closed groups'
+    experts lose even to negative choice scores; ties go to the lower index; weights sum to the scale."""
+    _skip(dev)
+    from mxserve.ops import seqmix
+
+    def route(s, c, k, groups, keep, scale=2.0, renorm=True):
+        z = torch.tensor([[_logit(x) for x in s]], device=dev)
+        w, ids = seqmix.route_topk(z, k, renorm, correction=torch.tensor(c, device=dev), groups=groups, keep=keep, scale=scale)
+        return w[0].double().cpu().numpy(), ids[0].cpu().tolist()
+
+    # group 0 has the single best expert, group 1 the better pair
+    s = [0.9, 0.1, 0.1, 0.6, 0.7, 0.2]
+    w, ids = route(s, [0.0] * 6, 2, 2, 1)
+    assert ids == [4, 3] and np.allclose(w, np.array([0.7, 0.6]) / 1.3 * 2.0, atol=1e-6)
+    # a correction brings group 0 ahead; the weights are the plain scores
+    w, ids = route(s, [0.0, 0.9, 0.0, 0.0, 0.0, 0.0], 2, 2, 1)
+    assert ids == [1, 0] and np.allclose(w, np.array([0.1, 0.9]) / 1.0 * 2.0, atol=1e-6)
+    # the kept group's choice scores are negative; the other group's third best would beat them
+    w, ids = route([0.5, 0.5, 0.5, 0.6, 0.6, 0.5], [-0.9, -0.95, -5.0, -0.2, -3.0, -2.0], 3, 2, 1)
+    assert ids == [0, 1, 2]
+    # without groups the same scores choose across
+    w, ids = route([0.5, 0.5, 0.5, 0.6, 0.6, 0.5], [-0.9, -0.95, -5.0, -0.2, -3.0, -2.0], 3, 1, 1)
+    assert ids == [3, 0, 1]
+    # ties, in groups and in experts
+    w, ids = route([0.5] * 8, [0.0] * 8, 3, 4, 2)
+    assert ids == [0, 1, 2] and np.allclose(w.sum(), 2.0)
+    # groups of one expert: its score alone
+    w, ids = route([0.2, 0.8, 0.4], [0.0] * 3, 2, 3, 2, scale=1.0, renorm=False)
+    assert ids == [1, 2] and np.allclose(w, [0.8, 0.4], atol=1e-6)
+    # all scores nearly zero: the sum is divided by, not floored
+    z = torch.full((1, 4), -60.0, device=dev)
+    w, _ = seqmix.route_topk(z, 2, True, correction=torch.zeros(4, device=dev), groups=2, keep=1, scale=1.0)
+    sc = 1.0 / (1.0 + math.exp(60.0))
+    assert np.allclose(w.double().cpu().numpy(), sc / (2 * sc + 1e-20), rtol=1e-4)
+
+
+@pytest.mark.parametrize("dev", DEVS)
+def test_routing_matches_the_oracle(dev):
+    _skip(dev)
+    from mxserve.ops import seqmix
+    g = torch.Generator().manual_seed(6)
+    for E, k, n, keep in ((12, 3, 4, 2), (64, 8, 8, 3), (6, 1, 1, 1), (200, 10, 10, 4), (130, 5, 65, 9)):
+        z, c = 2.0 * torch.randn(40, E, generator=g), 0.3 * torch.randn(E, generator=g)
+        w, ids = seqmix.route_topk(z.to(dev), k, True, correction=c.to(dev), groups=n, keep=keep, scale=1.7)
+        r = {"experts": E, "top": k, "groups": {"count": n, "keep": keep}, "scale": 1.7}
+        for t in range(40):
+            e, wt, margin = ao.choose_experts(z[t].double().numpy(), c.double().numpy(), r)
+            if margin > 1e-5:
+                assert ids[t].cpu().tolist() == e.tolist() and np.allclose(w[t].double().cpu().numpy(), wt, atol=1e-5)
+
+
+# ----------------------------------------------------------------------------- the streams
+@pytest.mark.parametrize("dev,dtype", DEV_DTYPE)
+@pytest.mark.parametrize("n,W", [(1, 64), (2, 96), (3, 37), (4, 260), (6, 48), (2, 12800), (9, 30)])
+def test_streams_alone(dev, dtype, n, W):
+    """Every stream from the old ones at once, the mix indexed [from, to] (not symmetric), bias and scale of the
+    sublayer's output, the next input's norm; row widths of whole pieces and others, and wider than a row buffer."""
+    _skip(dev)
+    from mxserve.ops import seqmix
+    g = torch.Generator().manual_seed(n * W)
+    T, V = 5, 11
+    rb = lambda *s: torch.randn(*s, generator=g).to(dtype)  # noqa: E731
+    table, y, bias, scale, nw1, nw2 = rb(V, W), rb(T, W), rb(W), rb(W), 0.1 * rb(W), 0.1 * rb(W)
+    w_in, w_in2, w_out, mix = (torch.randn(*s, generator=g) for s in ((n,), (n,), (n,), (n, n)))
+    ids = torch.tensor([3, 0, 10, 3, 7])
+    X, h = seqmix.streams_start(ids.to(dev), table.to(dev), n, w_in.to(dev), nw1.to(dev), EPS, 1.0, dtype)
+    d64 = lambda t: t.double().cpu().numpy()  # noqa: E731
+    tol = 1e-5 if dtype == torch.float32 else 0.02
+    Xn = np.stack([np.tile(d64(table)[i], (n, 1)) for i in ids.tolist()])
+    u = lambda x, w: np.stack([ao.streams_in(a, d64(w)) for a in x])  # noqa: E731
+    rel = lambda a, b: np.abs(a - b).max() / np.abs(b).max()  # noqa: E731
+    assert rel(d64(X), Xn) == 0.0 and rel(d64(h), ao.offset_norm(u(Xn, w_in), d64(nw1), EPS)) < tol
+    cf = torch.cat([mix.reshape(-1), w_out, w_in2])
+    for b, s in ((bias, scale), (None, scale), (None, None)):
+        dd = (d64(y) + (d64(b) if b is not None else 0.0)) * (d64(s) if s is not None else 1.0)
+        Xn = np.stack([ao.streams_out(x, d64(mix), d64(w_out), v) for x, v in zip(Xn, dd)])
+        h = seqmix.streams_update(X, y.to(dev), cf.to(dev), EPS, nw2.to(dev), dtype, bias=None if b is None else b.to(dev),
+                                  scale=None if s is None else s.to(dev), w_offset=1.0)
+        assert rel(d64(X), Xn) < 1e-5
+        assert rel(d64(h), ao.offset_norm(u(Xn, w_in2), d64(nw2), EPS)) < tol
+    if n > 1:
+        assert rel(np.stack([ao.streams_out(x, d64(mix).T, d64(w_out), v) for x, v in zip(Xn, dd)]),
+                   np.stack([ao.streams_out(x, d64(mix), d64(w_out), v) for x, v in zip(Xn, dd)])) > 0.05
+
+
+# ----------------------------------------------------------------------------- whole models, schedules
+@pytest.fixture(scope="module")
+def base(tmp_path_factory):
+    path = tmp_path_factory.mktemp("tarorax_base")
+    w = write_checkpoint(path, BASE, seed=11)
+    toks = {f"r{i}": _tokens(n, BASE["vocab"], 20 + i) for i, n in enumerate([90, 37, 1, 64, 130, 16])}
+    want = {rid: _oracle_model(BASE, w, t) for rid, t in toks.items()}
+    return path, w, toks, want
+
+
+@pytest.mark.parametrize("dev,dtype,tol", DEV_DTYPE_TOL)
+def test_portions_and_decoding(base, dev, dtype, tol):
+    """Whole prompt, token by token, and portions of several sizes down to two tokens (shorter than the filters)."""
+    _skip(dev)
+    path, _, toks, want = base
+    eng = engine(path, dev, dtype, max_tokens=256)
+    for sizes in ([1000], [1], [2], [40, 1], [3, 16, 2, 17, 1, 32, 5]):
+        steps = [[("a", p, False)] for p in cut(toks["r0"], sizes)]
+        steps[-1] = [("a", steps[-1][0][1], True)]
+        _check(replay(eng, steps)["a"], want["r0"][0], tol, want["r0"][1])
+    assert eng.kv.num_free() == eng.kv.num_blocks
+
+
+@pytest.mark.parametrize("dev,dtype,tol", DEV_DTYPE_TOL)
+def test_long_decoding(base, dev, dtype, tol):
+    """A short prompt, then well over a hundred tokens one by one (through the decode graphs on the GPU): pages
+    fill, new ones start, filters and states are carried all the way."""
+    _skip(dev)
+    path, _, toks, want = base
+    eng = engine(path, dev, dtype, max_tokens=192, eager=(dev == "cpu"))
+    steps = [[("a", p, False)] for p in cut(toks["r4"], [10, 1])]
+    steps[-1] = [("a", steps[-1][0][1], True)]
+    _check(replay(eng, steps)["a"], want["r4"][0], tol, want["r4"][1])
+    assert eng.kv.num_free() == eng.kv.num_blocks
+
+
+@pytest.mark.parametrize("dev,dtype,tol", DEV_DTYPE_TOL)
+@pytest.mark.parametrize("eager", [True, False])
+def test_mixed_batches_reuse_pages_and_slots(base, dev, dtype, tol, eager):
+    """Six unequal requests through four rows and a pool that cannot hold them all at once: portions of some beside
+    single tokens of others; each must equal the request run alone (the oracle)."""
+    _skip(dev)
+    if dev == "cpu" and not eager:
+        pytest.skip("graphs are a GPU path")
+    path, _, toks, want = base
+    eng = engine(path, dev, dtype, max_tokens=384, eager=eager)
+    rng = np.random.default_rng(3)
+    at = {r: 0 for r in toks}
+    waiting, live, steps = list(toks), [], []
+    while waiting or live:
+        while waiting and len(live) < 4 and sum(-(-len(toks[r]) // 64) * 64 for r in live + waiting[:1]) <= 384:
+            live.append(waiting.pop(0))
+        step = []
+        for r in list(live):
+            if rng.random() < 0.2 and len(live) > 1:
+                continue  # left out of this step
+            left = len(toks[r]) - at[r]
+            n = min(left, int(rng.choice([1, 1, 2, 3, 16, 29])))
+            end = n == left
+            step.append((r, toks[r][at[r]:at[r] + n], end))
+            at[r] += n
+            if end:
+                live.remove(r)
+        if step:
+            steps.append(step)
+    got = replay(eng, steps)
+    for r in toks:
+        _check(got[r], want[r][0], tol, want[r][1])
+    assert eng.kv.num_free() == eng.kv.num_blocks and not eng.runner._row_of
+
+
+@pytest.mark.parametrize("dev,dtype,tol", DEV_DTYPE_TOL)
+def test_request_that_fills_the_pool(tmp_path, dev, dtype, tol):
+    """A request three tokens short of the pool and of the longest sequence the engine admits: its last portions end
+    in partial tiles on the last page of the block table."""
+    _skip(dev)
+    cfg = config([layer(diff_attention(heads=4, kv_heads=2, dim=32, vdim=48, scale=0.15, conv=4), dense(128)),
+                  layer(gla(heads=4, dim=32, vdim=32, tau=16.0), moe(experts=4, top=2, ff=32, groups=2, keep=2)),
+                  layer(diff_attention(heads=8, kv_heads=1, dim=16, vdim=16, conv=2), None)], width=128, vocab=200, streams=2)
+    w = write_checkpoint(tmp_path, cfg, seed=8)
+    t = _tokens(125, cfg["vocab"], 9)
+    want, margins = _oracle_model(cfg, w, t)
+    eng = engine(tmp_path, dev, dtype, max_tokens=128)
+    for sizes in ([1000], [90, 35], [100, 19, 1], [64, 40, 21]):
+        steps = [[("a", p, False)] for p in cut(t, sizes)]
+        steps[-1] = [("a", steps[-1][0][1], True)]
+        _check(replay(eng, steps)["a"], want, tol, margins)
+    assert eng.kv.num_free() == eng.kv.num_blocks
+
+
+VARIANTS = {
+    "one_of_everything": config([layer(diff_attention(heads=1, kv_heads=1, dim=1, vdim=1, conv=1, every=1), dense(1)),
+                                 layer(gla(heads=1, dim=1, vdim=1, tau=1.0), moe(experts=1, top=1, ff=1, groups=1, keep=1, scale=1.0))],
+                                width=40, vocab=50, streams=1, eps=1e-3),
+    "recurrent_layers_only": config([layer(gla(), None), layer(gla(heads=1, dim=64, vdim=8, tau=2.0), dense(33))], width=64, vocab=70, streams=2),
+    "attention_layers_only": config([layer(diff_attention(), None), layer(diff_attention(heads=2, kv_heads=1, dim=8, vdim=8, softcap=80.0,
+                                                                                        conv=2), None)], width=64, vocab=70, streams=5),
+    "a_single_layer": config([layer(diff_attention(heads=2, kv_heads=1, dim=16, vdim=8, conv=7), moe(3, 1, 24, 3, 1))], width=32, vocab=33,
+                             streams=4),
+    "equal_sizes_everywhere": config([layer(diff_attention(heads=16, kv_heads=16, dim=16, vdim=16, scale=0.25, conv=16, every=16), dense(16)),
+                                      layer(gla(heads=16, dim=16, vdim=16, tau=16.0), moe(experts=16, top=16, ff=16, groups=16, keep=16))],
+                                     width=16, vocab=16, streams=2),
+    "sizes_that_fit_no_vector_load": config([layer(diff_attention(heads=3, kv_heads=1, dim=5, vdim=7, conv=3), moe(6, 2, 14, 3, 2)),
+                                             layer(gla(heads=5, dim=6, vdim=9), dense(22))], width=50, vocab=37, streams=3),
+    "wide_heads": config([layer(diff_attention(heads=6, kv_heads=3, dim=72, vdim=136, scale=0.07, conv=4), moe(9, 2, 40, 3, 2)),
+                          layer(gla(heads=2, dim=144, vdim=72), dense(100))], width=72, vocab=60, streams=2),
+}
+
+
+@pytest.mark.parametrize("dev,dtype,tol", DEV_DTYPE_TOL)
+@pytest.mark.parametrize("name", list(VARIANTS))
+def test_other_sizes(tmp_path, dev, dtype, tol, name):
+    _skip(dev)
+    cfg = VARIANTS[name]
+    w = write_checkpoint(tmp_path, cfg, seed=5)
+    t = _tokens(45, cfg["vocab"], 6)
+    want, margins = _oracle_model(cfg, w, t)
+    eng = engine(tmp_path, dev, dtype, max_tokens=128)
+    for sizes in ([1000], [20, 2, 1, 7, 1]):
+        steps = [[("a", p, False)] for p in cut(t, sizes)]
+        steps[-1] = [("a", steps[-1][0][1], True)]
+        if name == "one_of_everything" and tol > 1e-2:
+            # a head of one value is its own unit norm: only its sign is left, which rounding may turn
+            assert np.isfinite(replay(eng, steps)["a"]).all()
+        else:
+            _check(replay(eng, steps)["a"], want, tol, margins)
+
+
+@pytest.mark.parametrize("dev", DEVS)
+def test_layer_tap_matches_oracle_streams(base, dev):
+    """The sum of the streams after every layer, layer by layer."""
+    _skip(dev)
+    path, w, toks, _ = base
+    eng = engine(path, dev, "float32", max_tokens=128)
+    tap = eng.runner.model.layer_tap = []
+    replay(eng, [[("a", toks["r1"], True)]])
+    ref = ao.run(BASE, w, toks["r1"])[1]
+    assert len(tap) == len(ref) == len(BASE["layers"])
+    for a, b in zip(tap, ref):
+        assert np.abs(a.double().cpu().numpy() - b).max() < 1e-3 * max(1.0, np.abs(b).max())
+
+
+def test_pages_slots_and_tensors_of_the_plan():
+    """An attention layer pages two keys and a value per kv head and keeps its filter's inputs in the slot, a gated
+    linear layer keeps its matrix there; every layer has places of its own."""
+    from mxserve.models.config import tarorax_config
+    from mxserve.models.tarorax import layer_plan, weight_shapes
+    plan = layer_plan(BASE, 16)
+    per_token = [l["mixer"]["kv_heads"] * (2 * l["mixer"]["dim"] + l["mixer"]["vdim"]) for l in BASE["layers"] if l["type"] == "attention"]
+    floats = []
+    for l in BASE["layers"]:
+        mc = l["mixer"]
+        if l["type"] == "gla":
+            floats.append(mc["heads"] * mc["dim"] * mc["vdim"])
+        else:
+            floats.append((mc["conv"] - 1) * (2 * mc["heads"] * mc["dim"] + mc["kv_heads"] * (2 * mc["dim"] + mc["vdim"])))
+    assert plan.block_elems == 16 * sum(per_token)
+    assert plan.state_floats == sum(-(-f // 4) * 4 for f in floats) and len({r.soff for r in plan.runs}) == len(plan.runs)
+    sh = weight_shapes(BASE)
+    assert sh["l0.hc2.mix"] == (3, 3) and sh["l0.hc1.in"] == (3,) and "l2.hc2.mix" not in sh and "l2.ls2" not in sh
+    assert sh["l1.mix.q"] == (2 * 6 * 24, BASE["width"]) and sh["l1.mix.k.conv"] == (2 * 2 * 24, 3) and sh["l1.mix.lk2"] == (24,)
+    assert sh["l3.mlp.correction"] == (6,) and "l3.mlp.e0.gate" not in sh and "head" not in sh
+    cfg = tarorax_config("m", BASE)
+    assert cfg.has_recurrent_state and cfg.kv_bytes_per_token(2) == 2 * sum(per_token)
+
+
+@pytest.mark.parametrize("dev,dtype", [("cpu", "float32"), pytest.param("cuda", "float32", marks=pytest.mark.gpu),
+                                       pytest.param("cuda", "bfloat16", marks=pytest.mark.gpu)])
+def test_greedy_generation_through_the_scheduler(base, dev, dtype):
+    """LLMEngine.generate: the scheduler chunks the prompts (a small token budget), batches the requests and
+    decodes; every generated token must be the oracle's choice given the same prefix (or within its near-ties)."""
+    _skip(dev)
+    from mxserve.config import EngineArgs
+    from mxserve.engine.engine import LLMEngine
+    from mxserve.engine.request import SamplingParams
+    path, w, toks, _ = base
+    args = EngineArgs(model=str(path), device=dev, dtype=dtype, num_gpu_blocks=40, cpu_num_blocks=40, max_model_len=256,
+                      max_num_seqs=3, max_num_batched_tokens=48, load_format="safetensors", cuda_graph_max_bs=2)
+    eng = LLMEngine(args)
+    assert not eng.kv.caching  # a cached page has no state to go on from
+    prompts = [toks["r1"], toks["r3"], toks["r2"], toks["r5"], toks["r3"][:40] + toks["r5"]]
+    outs = eng.generate(prompts, SamplingParams(max_tokens=12, temperature=0.0, ignore_eos=True))
+    margin = 1e-3 if dtype == "float32" else 0.25
+    for p, o in zip(prompts, outs):
+        assert len(o) == 12
+        lg = ao.run(BASE, w, p + o[:-1])[0][len(p) - 1:]
+        for row, tok in zip(lg, o):
+            assert row[tok] >= row.max() - margin * (row.max() - row.min())
+
+
+def test_registered_small_model_runs():
+    """The registry's small Tarorax with random weights, by name, as a served model would start."""
+    from mxserve.config import EngineArgs
+    from mxserve.engine.engine import LLMEngine
+    from mxserve.engine.request import SamplingParams
+    eng = LLMEngine(EngineArgs(model="tiny-tarorax", device="cpu", dtype="float32", num_gpu_blocks=16, cpu_num_blocks=16,
+                               max_model_len=128, max_num_seqs=2, max_num_batched_tokens=64))
+    outs = eng.generate([[1, 2, 3, 4, 5], [7] * 20], SamplingParams(max_tokens=5, temperature=0.0, ignore_eos=True))
+    assert [len(o) for o in outs] == [5, 5]
+
+
+def test_trace_runner_command_line(base, tmp_path):
+    """bin/trace_run as a user starts it: steps on stdin, `done <step>` after each, logits files for the steps that
+    want some, pages and slots given back under --max-tokens."""
+    import json
+    import os
+    import subprocess
+    import sys
+    path, _, toks, want = base
+    root = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
+    t = toks["r1"]
+    steps = [{"step": 0, "entries": [{"id": "x", "tokens": t[:20], "want": [0, 19]}], "end": []},
+             {"step": 1, "entries": [{"id": "x", "tokens": t[20:22], "want": []}, {"id": "y", "tokens": toks["r2"], "want": [0]}],
+              "end": ["y"]},
+             {"step": 2, "entries": [{"id": "x", "tokens": t[22:], "want": [len(t) - 23]}], "end": ["x"]}]
+    out = tmp_path / "out"
+    r = subprocess.run([sys.executable, os.path.join(root, "bin", "trace_run"), "--model", str(path), "--dtype", "float32",
+                        "--out", str(out), "--max-tokens", "128", "--device", "cpu"],
+                       input="\n".join(json.dumps(s) for s in steps) + "\n", capture_output=True, text=True, timeout=300)
+    assert r.returncode == 0, r.stderr[-2000:]
+    assert [l for l in r.stdout.splitlines() if l.startswith("done")] == ["done 0", "done 1", "done 2"]
+    V = BASE["vocab"]
+    a = np.fromfile(out / "0.f32", dtype="<f4").reshape(-1, V)
+    b = np.fromfile(out / "1.f32", dtype="<f4").reshape(-1, V)
+    c = np.fromfile(out / "2.f32", dtype="<f4").reshape(-1, V)
+    _check(a.astype(np.float64), want["r1"][0][[0, 19]], 1e-4)
+    _check(b.astype(np.float64), want["r2"][0][[0]], 1e-4)
+    _check(c.astype(np.float64), want["r1"][0][[len(t) - 1]], 1e-4)
