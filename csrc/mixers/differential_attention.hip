@@ -66,10 +66,10 @@ __device__ __forceinline__ Bound make_bound(float scale, float cap) {
 }
 
 template <int KSM, int VTM, int NQ, int NK, bool ONLINE>
-__global__ void __launch_bounds__(512, 2) differential_attention_mfma_kernel(const DiffArgs p) {
+__global__ void __launch_bounds__(128 * NQ * NK, 2) differential_attention_mfma_kernel(const DiffArgs p) {
   constexpr int KSUB = NK == 1 ? 2 : 1;      // 32-key runs a wave takes of a tile
   constexpr int KT = 32 * KSUB * NK;         // keys per tile
-  constexpr int NT = 512;
+  constexpr int NW = 2 * NQ * NK, NT = 64 * NW;
   constexpr int KP = (KT * 4 * KSM + NT - 1) / NT;         // 16-byte key pieces per thread (two maps of 16 KSM elements)
   constexpr int VP = (KT / 4 * 8 * VTM + NT - 1) / NT;     // 4 keys x 4 columns value units per thread
   constexpr bool PRE = !(VTM == 8 && NK > 1);              // next tile's loads wait in registers
@@ -80,17 +80,18 @@ __global__ void __launch_bounds__(512, 2) differential_attention_mfma_kernel(con
   const int KLD = KS * 16 + 8;               // padded LDS row of a key
   bf16_t* ks = reinterpret_cast<bf16_t*>(smem);            // [2][KT][KLD]
   bf16_t* vs = ks + 2 * KT * KLD;                          // [32 VT][VLD]
-  float* xch = reinterpret_cast<float*>(smem);             // [8 waves][32][40], after the walk
-  __shared__ float wsum[8][32], wmax[ONLINE ? 8 : 1][32];
+  float* xch = reinterpret_cast<float*>(smem);             // [NW][32][40], after the walk
+  __shared__ float wsum[NW][32], wmax[ONLINE ? NW : 1][32];
   const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6;
   const int c = lane & 31, hl = lane >> 5;
   // wave = map + 2 * (column group * NK + key group)
   const int map = wid & 1, wk = (wid >> 1) % NK, wq = (wid >> 1) / NK;
-  const int s = blockIdx.z / p.nsplit, sp = blockIdx.z - s * p.nsplit, g = blockIdx.y;
+  const int s = blockIdx.z / p.nsplit, sp = blockIdx.z - s * p.nsplit, g = blockIdx.x;
   const int row0 = p.qsl[s];
   const int qlen = min(p.qsl[s + 1], p.n_rows) - row0;
   const int rep = p.H / p.G;
-  const int c0 = (static_cast<int>(gridDim.x) - 1 - static_cast<int>(blockIdx.x)) * 32 * NQ;  // long walks first
+  // long walks first, the kv heads' workgroups of one tile side by side
+  const int c0 = (static_cast<int>(gridDim.y) - 1 - static_cast<int>(blockIdx.y)) * 32 * NQ;
   if (row0 < 0 || qlen <= 0 || c0 >= qlen * rep) return;  // workgroup-uniform
   // the chunk's first position; its last row stays inside the block table whatever the metadata says
   const int pos0 = min(max(p.seq_lens[s] - qlen, 0), max(p.bt_stride * 16 - qlen, 0));
@@ -554,7 +555,7 @@ static bool launch_mfma(const DiffArgs& a, int S, hipStream_t st) {
   constexpr int KT = 32 * (NK == 1 ? 2 : 1) * NK;
   const int KS = (a.dk + 15) / 16, VT = (a.dv + 31) / 32;
   const size_t stage = 2 * static_cast<size_t>(2 * KT * (KS * 16 + 8) + 32 * VT * (KT + 8));
-  const size_t shm = std::max<size_t>(stage, 8 * 32 * 40 * sizeof(float));
+  const size_t shm = std::max<size_t>(stage, 2 * NQ * NK * 32 * 40 * sizeof(float));
   if (shm > 64 * 1024 - 4096) {
     if (hipFuncSetAttribute(reinterpret_cast<const void*>(&differential_attention_mfma_kernel<KSM, VTM, NQ, NK, ONLINE>),
                             hipFuncAttributeMaxDynamicSharedMemorySize, 156 * 1024) != hipSuccess) {
@@ -563,9 +564,9 @@ static bool launch_mfma(const DiffArgs& a, int S, hipStream_t st) {
     }
   }
   const int cols = a.max_q * (a.H / a.G);
-  const dim3 grid((cols + 32 * NQ - 1) / (32 * NQ), a.G, S * a.nsplit);
+  const dim3 grid(a.G, (cols + 32 * NQ - 1) / (32 * NQ), S * a.nsplit);
   if (grid.z > 65535u || grid.y > 65535u) return false;
-  hipLaunchKernelGGL((differential_attention_mfma_kernel<KSM, VTM, NQ, NK, ONLINE>), grid, dim3(512), shm, st, a);
+  hipLaunchKernelGGL((differential_attention_mfma_kernel<KSM, VTM, NQ, NK, ONLINE>), grid, dim3(128 * NQ * NK), shm, st, a);
   MXS_CHECK_LAUNCH();
   return true;
 }
